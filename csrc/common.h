@@ -81,6 +81,27 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   return t;
 }
 
+// one step of a sum over neighbouring lanes as a data-parallel-primitive add (no trip through LDS)
+template <int CTRL> __device__ __forceinline__ float dpp_add(float v) {
+  return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
+}
+
+// sum over the P row parts of a wave, every lane gets it.  NEAR: the parts of a column are P neighbouring lanes
+// (lane = column * P + part): swaps inside quads, then mirrors of 8 and 16 lanes.  Otherwise the parts are 64 / P
+// lanes apart (lane = part * (64 / P) + column): xor-shuffles.
+template <int P, bool NEAR> __device__ __forceinline__ float parts_sum(float v) {
+  if constexpr (NEAR) {
+    v = dpp_add<0xB1>(v);                           // quad_perm [1, 0, 3, 2]
+    v = dpp_add<0x4E>(v);                           // quad_perm [2, 3, 0, 1]
+    if constexpr (P >= 8) v = dpp_add<0x141>(v);    // row_half_mirror
+    if constexpr (P >= 16) v = dpp_add<0x140>(v);   // row_mirror
+  } else {
+#pragma unroll
+    for (int o = 64 / P; o < 64; o <<= 1) v += __shfl_xor(v, o, 64);
+  }
+  return v;
+}
+
 #define HIP_LAUNCH_CHECK()                                  \
   do {                                                      \
     hipError_t e_ = hipGetLastError();                      \

@@ -1,8 +1,8 @@
-// The gated delta rule with a decay per head and key channel and a per-request fp32 state, gfx950.  Compiled without
+// The gated delta rule with a decay per head and key channel (or per head) and a per-request fp32 state, gfx950.  Compiled without
 // fast-math: everything that enters the recurrence is 32-bit by definition of such a model.
 //
 //   delta_rule_prep   per row: q and k of every query / key head made unit vectors (q times dim^-0.5), the decays
-//                     g = exp(-exp(a_log[h]) * softplus(dt + dt_bias)) per head and key channel, b = sigmoid(beta),
+//                     g = exp(-exp(a_log[h]) * softplus(dt + dt_bias)) per head (and key channel), b = sigmoid(beta),
 //                     k.q of the unit vectors;
 //                     all fp32, computed once per row instead of once per lane of the recurrence
 //   gated_delta_rule  per (sequence, head, tile of 16 to 64 value columns) a workgroup walks the sequence's rows:
@@ -32,7 +32,8 @@ template <typename F> int by_dtype(int dt, F&& f) {
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
 // grid (rows): waves of the block take the units in turn - G query heads, G key heads (a wave each: sum of squares
-// over dim), then the H * dim decays and H betas element by element.
+// over dim), then the decays and the H betas element by element.  decay null: one decay per head (dt and dt_bias have H
+// columns), kept as the third row of bsig [T, 3, H]; else H * dim decays and bsig [T, 2, H].
 template <typename T>
 __global__ __launch_bounds__(256) void delta_rule_prep_kernel(float* __restrict__ qn, float* __restrict__ kn,
                                                               float* __restrict__ decay, float* __restrict__ bsig,
@@ -45,6 +46,7 @@ __global__ __launch_bounds__(256) void delta_rule_prep_kernel(float* __restrict_
   const long t = blockIdx.x;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nwaves = blockDim.x >> 6;
   const T* xr = x + t * x_stride;
+  const int nb = decay != nullptr ? 2 : 3;
   const float qscale = 1.0f / sqrtf((float)dim);
   for (int g = wave; g < G; g += nwaves) {          // [q heads | k heads], each dim wide
     const T* qs = xr + (long)g * dim;
@@ -63,35 +65,18 @@ __global__ __launch_bounds__(256) void delta_rule_prep_kernel(float* __restrict_
     }
     dot = wave_sum(dot);
     const int per = H / G;
-    for (int j = lane; j < per; j += 64) bsig[t * 2 * H + H + g * per + j] = dot;
+    for (int j = lane; j < per; j += 64) bsig[t * nb * H + H + g * per + j] = dot;
   }
   const T* dr = dt + t * dt_stride;
-  for (int i = threadIdx.x; i < H * dim; i += blockDim.x) {
-    const int h = i / dim;
-    decay[t * (long)H * dim + i] = expf(-expf(a_log[h]) * softplus_f(ldf(dr + i) + dt_bias[i]));
+  if (decay != nullptr)
+    for (int i = threadIdx.x; i < H * dim; i += blockDim.x) {
+      const int h = i / dim;
+      decay[t * (long)H * dim + i] = expf(-expf(a_log[h]) * softplus_f(ldf(dr + i) + dt_bias[i]));
+    }
+  for (int h = threadIdx.x; h < H; h += blockDim.x) {
+    bsig[t * nb * H + h] = 1.0f / (1.0f + expf(-ldf(beta + t * beta_stride + h)));
+    if (decay == nullptr) bsig[t * 3 * H + 2 * H + h] = expf(-expf(a_log[h]) * softplus_f(ldf(dr + h) + dt_bias[h]));
   }
-  for (int h = threadIdx.x; h < H; h += blockDim.x) bsig[t * 2 * H + h] = 1.0f / (1.0f + expf(-ldf(beta + t * beta_stride + h)));
-}
-
-// one step of a sum over neighbouring lanes as a data-parallel-primitive add (no trip through LDS)
-template <int CTRL> __device__ __forceinline__ float dpp_add(float v) {
-  return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
-}
-
-// sum over the P row parts of a wave, every lane gets it.  NEAR: the parts of a column are P neighbouring lanes
-// (lane = column * P + part): swaps inside quads, then mirrors of 8 and 16 lanes.  Otherwise the parts are 64 / P
-// lanes apart (lane = part * (64 / P) + column): xor-shuffles.
-template <int P, bool NEAR> __device__ __forceinline__ float parts_sum(float v) {
-  if constexpr (NEAR) {
-    v = dpp_add<0xB1>(v);                           // quad_perm [1, 0, 3, 2]
-    v = dpp_add<0x4E>(v);                           // quad_perm [2, 3, 0, 1]
-    if constexpr (P >= 8) v = dpp_add<0x141>(v);    // row_half_mirror
-    if constexpr (P >= 16) v = dpp_add<0x140>(v);   // row_mirror
-  } else {
-#pragma unroll
-    for (int o = 64 / P; o < 64; o <<= 1) v += __shfl_xor(v, o, 64);
-  }
-  return v;
 }
 
 // grid (tiles of CB = 4 * 64 / P value columns, H, sequences), 4 waves: wave w owns columns w * 64 / P .. of the tile,
@@ -104,9 +89,11 @@ template <int P, bool NEAR> __device__ __forceinline__ float parts_sum(float v) 
 // the head, fp32), v (the tile's columns), b and k.q of a chunk are staged in LDS by the whole workgroup - the next
 // chunk's loads are in flight while the current one is computed, one barrier per chunk - and read back as broadcasts
 // (16-byte reads: a group of four rows).
+// PH: one decay per head and row: it is not staged per key channel, and r and p are summed over the undecayed state and
+// multiplied by it afterwards.
 // x rows hold v (H * vdim) at column v_off; qn / kn [T, G, dim], decay [T, H, dim], bsig [T, 2, H] (sigmoid(beta), then
-// k.q of the head's group) fp32; out [T, H * vdim] fp32; state [slots, H, dim, vdim] fp32.
-template <typename T, int R, int C, int P, bool NEAR>
+// k.q of the head's group) or, PH, [T, 3, H] (and the decay) fp32; out [T, H * vdim] fp32; state [slots, H, dim, vdim] fp32.
+template <typename T, int R, int C, int P, bool NEAR, bool PH>
 __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict__ out, const T* __restrict__ x,
                                                                long x_stride, int v_off, const float* __restrict__ qn,
                                                                const float* __restrict__ kn,
@@ -117,7 +104,9 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict
                                                                int vdim) {
   constexpr int CT = 64 / P, CB = 4 * CT;           // columns per wave, per workgroup
   constexpr int DP = P * R;                         // rows, padded (rows past dim stay zero)
-  constexpr int ROW = 3 * DP + CB + 4;              // floats staged per sequence row: q | k | g | v (CB) | b, k.q, pad
+  constexpr int VO = (PH ? 2 : 3) * DP;
+  constexpr int ROW = VO + CB + 4;                  // floats staged per sequence row: q | k | g (not PH) | v (CB) | b, k.q, g
+  constexpr int NB = PH ? 3 : 2;
   __shared__ __attribute__((aligned(16))) float lds[2][C * ROW];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int cl = NEAR ? lane / P : lane & (CT - 1), part = NEAR ? lane & (P - 1) : lane / CT;
@@ -141,13 +130,13 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict
   // staging: a thread brings 16 bytes of q, of k and of g per pass (all of one row), v and b / k.q element by element
   constexpr int F4 = DP / 4;                        // 16-byte pieces per row and array (a power of two)
   constexpr int NQ = (C * F4 + 255) / 256, NV = (C * CB + 255) / 256;
-  static_assert(2 * C <= 256, "b and k.q of a chunk are one pass");
+  static_assert(NB * C <= 256, "b, k.q and g of a chunk are one pass");
   const bool vec = (dim & 3) == 0;                  // (rows of qn / kn / decay start on 16-byte borders)
   const float* qsrc = qn + ((long)q0 * G + g) * dim;
   const float* ksrc = kn + ((long)q0 * G + g) * dim;
-  const float* gsrc = decay + ((long)q0 * H + h) * dim;
+  const float* gsrc = PH ? nullptr : decay + ((long)q0 * H + h) * dim;
   const T* vsrc = x + (long)q0 * x_stride + v_off + (long)h * vdim + col0;
-  const float* bsrc = bsig + (long)q0 * 2 * H + h;
+  const float* bsrc = bsig + (long)q0 * NB * H + h;
   const long qstep = (long)G * dim, gstep = (long)H * dim;
   f32x4 sq[NQ], sk[NQ], sg[NQ];
   float sv[NV], sb = 0.f;
@@ -170,7 +159,7 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict
       if (j < rows) {
         sq[e] = piece(qsrc + (first + j) * qstep, f);
         sk[e] = piece(ksrc + (first + j) * qstep, f);
-        sg[e] = piece(gsrc + (first + j) * gstep, f);
+        if constexpr (!PH) sg[e] = piece(gsrc + (first + j) * gstep, f);
       }
     }
 #pragma unroll
@@ -178,7 +167,7 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict
       const int idx = tid + e * 256, j = idx / CB, cc = idx & (CB - 1);
       sv[e] = (j < rows && col0 + cc < vdim) ? ldf(vsrc + (first + j) * x_stride + cc) : 0.f;
     }
-    sb = (tid < 2 * C && (tid >> 1) < rows) ? bsrc[(long)(first + (tid >> 1)) * 2 * H + (tid & 1) * H] : 0.f;
+    sb = (tid < NB * C && tid / NB < rows) ? bsrc[(long)(first + tid / NB) * NB * H + (tid % NB) * H] : 0.f;
   };
   auto stash = [&](int buf) {
     float* dst = lds[buf];
@@ -188,15 +177,15 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict
       if (j < C) {
         *reinterpret_cast<f32x4*>(dst + j * ROW + f) = sq[e];
         *reinterpret_cast<f32x4*>(dst + j * ROW + DP + f) = sk[e];
-        *reinterpret_cast<f32x4*>(dst + j * ROW + 2 * DP + f) = sg[e];
+        if constexpr (!PH) *reinterpret_cast<f32x4*>(dst + j * ROW + 2 * DP + f) = sg[e];
       }
     }
 #pragma unroll
     for (int e = 0; e < NV; ++e) {
       const int idx = tid + e * 256, j = idx / CB, cc = idx & (CB - 1);
-      if (j < C) dst[j * ROW + 3 * DP + cc] = sv[e];
+      if (j < C) dst[j * ROW + VO + cc] = sv[e];
     }
-    if (tid < 2 * C) dst[(tid >> 1) * ROW + 3 * DP + CB + (tid & 1)] = sb;
+    if (tid < NB * C) dst[tid / NB * ROW + VO + CB + tid % NB] = sb;
   };
   const int chunks = (n + C - 1) / C;
   fetch(0);
@@ -216,11 +205,14 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict
         const int off = ((i >> 2) * P + part) * 4;
         const f32x4 qv = *reinterpret_cast<const f32x4*>(L + off);
         const f32x4 kv = *reinterpret_cast<const f32x4*>(L + DP + off);
-        const f32x4 gv = *reinterpret_cast<const f32x4*>(L + 2 * DP + off);
+        f32x4 gv;
+        if constexpr (!PH) gv = *reinterpret_cast<const f32x4*>(L + 2 * DP + off);
 #pragma unroll
         for (int e = 0; e < 4; e += 2) {
-          S[i + e] *= gv[e];
-          S[i + e + 1] *= gv[e + 1];
+          if constexpr (!PH) {
+            S[i + e] *= gv[e];
+            S[i + e + 1] *= gv[e + 1];
+          }
           ra += S[i + e] * kv[e];
           rb += S[i + e + 1] * kv[e + 1];
           pa += S[i + e] * qv[e];
@@ -229,12 +221,17 @@ __global__ __launch_bounds__(256) void gated_delta_rule_kernel(float* __restrict
           kr[i + e + 1] = kv[e + 1];
         }
       }
-      const float r = parts_sum<P, NEAR>(ra + rb);
-      const float p = parts_sum<P, NEAR>(pa + pb);
-      const float u = L[3 * DP + CB] * (L[3 * DP + wave * CT + cl] - r);
+      float r = parts_sum<P, NEAR>(ra + rb);
+      float p = parts_sum<P, NEAR>(pa + pb);
+      const float gs = PH ? L[VO + CB + 2] : 1.f;
+      if constexpr (PH) { r *= gs; p *= gs; }
+      const float u = L[VO + CB] * (L[VO + wave * CT + cl] - r);
 #pragma unroll
-      for (int i = 0; i < R; ++i) S[i] += kr[i] * u;
-      if (part == 0 && col_ok) out[(long)(q0 + c * C + j) * H * vdim + (long)h * vdim + col] = p + L[3 * DP + CB + 1] * u;
+      for (int i = 0; i < R; ++i) {
+        if constexpr (PH) S[i] = gs * S[i] + kr[i] * u;
+        else S[i] += kr[i] * u;
+      }
+      if (part == 0 && col_ok) out[(long)(q0 + c * C + j) * H * vdim + (long)h * vdim + col] = p + L[VO + CB + 1] * u;
     }
     if (c + 1 < chunks) stash((c + 1) & 1);
     __syncthreads();
@@ -266,7 +263,7 @@ VDAMD_API int vdamd_delta_rule_prep(float* qn, float* kn, float* decay, float* b
 }
 
 // x [T, x_stride] of type dtype with v at column v_off; dim <= 256.  max_rows: the most rows any sequence brings (0 =
-// unknown).  parts: row parts per wave (4, 8 or 16; 0 = chosen here)
+// unknown).  parts: row parts per wave (4, 8 or 16; 0 = chosen here).  decay null: one decay per head, in bsig [T, 3, H]
 VDAMD_API int vdamd_gated_delta_rule(float* out, const void* x, long x_stride, int v_off, const float* qn,
                                      const float* kn, const float* decay, const float* bsig, float* state,
                                      const int* slots, const int* qsl, const int* seq_lens, int B, int H, int G, int dim,
@@ -288,9 +285,13 @@ VDAMD_API int vdamd_gated_delta_rule(float* out, const void* x, long x_stride, i
   const dim3 grid((vdim + 256 / parts - 1) / (256 / parts), H, B);
   const int rc = by_dtype(dtype, [&](auto* tp) {
     using TT = std::remove_pointer_t<decltype(tp)>;
-#define GDR(R_, P_)                                                                                                    \
-  hipLaunchKernelGGL((gated_delta_rule_kernel<TT, R_, 8, P_, (P_ >= 8)>), grid, dim3(256), 0, stream, out,             \
+#define GDR_H(R_, P_, PH_)                                                                                             \
+  hipLaunchKernelGGL((gated_delta_rule_kernel<TT, R_, 8, P_, (P_ >= 8), PH_>), grid, dim3(256), 0, stream, out,        \
                      (const TT*)x, x_stride, v_off, qn, kn, decay, bsig, state, slots, qsl, seq_lens, H, G, dim, vdim)
+#define GDR(R_, P_)                                                                    \
+  do {                                                                                 \
+    if (decay == nullptr) GDR_H(R_, P_, true); else GDR_H(R_, P_, false);              \
+  } while (0)
 #define GDR_P(P_)                                                        \
   do {                                                                   \
     if (r <= 4) GDR(4, P_); else if (r <= 8) GDR(8, P_);                 \
@@ -301,6 +302,7 @@ VDAMD_API int vdamd_gated_delta_rule(float* out, const void* x, long x_stride, i
     else GDR_P(16);
 #undef GDR_P
 #undef GDR
+#undef GDR_H
   });
   if (rc) return 1;
   HIP_LAUNCH_CHECK();

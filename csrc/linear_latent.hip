@@ -10,7 +10,7 @@
 //                            one head's S for one sequence, in registers (up to 16 waves x dim/16 rows each), and walks
 //                            the sequence's rows in chunks staged through LDS: prompt portions and single decoded rows
 //                            are the same kernel (launches of decoded rows only take small workgroups)
-//   gated_rms_norm           o / sqrt(mean(o^2) + eps) * w * sigmoid(g) * scale, over whole rows or over runs of `group`
+//   gated_rms_norm           o / sqrt(mean(o^2) + eps) * w * sigmoid(g) * scale (or silu(g)), over whole rows or over runs of `group`
 //                            values (heads) that share w
 //   clamped_glu              min(g, L) sigmoid(alpha min(g, L)) (clamp(u, -L, L) + 1) over [g | u]
 //   relu_squared             max(x, 0)^2
@@ -87,10 +87,13 @@ __global__ void layer_norm_kernel(TO* __restrict__ out, TX* __restrict__ x, long
     stf(orow + i, (ldf(xr + i) - mean) * inv * w[i] + (b != nullptr ? b[i] : 0.f));
 }
 
+// what multiplies a normed value: sigmoid(g), or g * sigmoid(g)
+__device__ __forceinline__ float gate_f(float g, int silu) { return silu ? g * sigmoid_f(g) : sigmoid_f(g); }
+
 template <typename TG, typename TO>
 __global__ void gated_rms_norm_kernel(TO* __restrict__ out, long out_stride, const float* __restrict__ o,
                                       const float* __restrict__ w, const TG* __restrict__ gate, long gate_stride,
-                                      float eps, int N, float scale) {
+                                      float eps, int N, float scale, int silu) {
   __shared__ float red[17];
   const long row = blockIdx.x;
   const float* orow = o + row * (long)N;
@@ -99,7 +102,7 @@ __global__ void gated_rms_norm_kernel(TO* __restrict__ out, long out_stride, con
   for (int i = threadIdx.x; i < N; i += blockDim.x) { const float f = orow[i]; ss += f * f; }
   const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)N + eps);
   TO* dst = out + row * out_stride;
-  for (int i = threadIdx.x; i < N; i += blockDim.x) stf(dst + i, orow[i] * inv * w[i] * sigmoid_f(ldf(g + i)) * scale);
+  for (int i = threadIdx.x; i < N; i += blockDim.x) stf(dst + i, orow[i] * inv * w[i] * gate_f(ldf(g + i), silu) * scale);
 }
 
 // the norm over runs of `group` values (one head each) that share w[group]: a wave per run, rows x runs of work
@@ -107,7 +110,7 @@ template <typename TG, typename TO>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(TO* __restrict__ out, long out_stride,
                                                                const float* __restrict__ o, const float* __restrict__ w,
                                                                const TG* __restrict__ gate, long gate_stride, float eps,
-                                                               int rows, int N, int group, float scale) {
+                                                               int rows, int N, int group, float scale, int silu) {
   const int lane = threadIdx.x & 63;
   const int per_row = N / group;
   const long unit = (long)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
@@ -120,7 +123,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(TO* __restrict__ 
   const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)group + eps);
   const TG* g = gate + row * gate_stride + c0;
   TO* dst = out + row * out_stride + c0;
-  for (int i = lane; i < group; i += 64) stf(dst + i, orow[i] * inv * w[i] * sigmoid_f(ldf(g + i)) * scale);
+  for (int i = lane; i < group; i += 64) stf(dst + i, orow[i] * inv * w[i] * gate_f(ldf(g + i), silu) * scale);
 }
 
 // the same for 16-bit gate and result and runs of 8 L values, L a power of two up to 64: L neighbouring lanes per run, 8
@@ -132,7 +135,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(T* __restrict
                                                                    const float* __restrict__ w,
                                                                    const T* __restrict__ gate, long gate_stride,
                                                                    float eps, long units, int N, int group, int L,
-                                                                   float scale) {
+                                                                   float scale, int silu) {
   using V8 = typename Vec8<T>::type;
   const long idx = (long)blockIdx.x * 256 + threadIdx.x;
   const long unit = idx / L;
@@ -154,7 +157,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(T* __restrict
   const float wf[8] = {wa.x, wa.y, wa.z, wa.w, wb.x, wb.y, wb.z, wb.w};
   V8 r;
 #pragma unroll
-  for (int e = 0; e < 8; ++e) r[e] = (T)(of[e] * inv * wf[e] * sigmoid_f((float)gv[e]));
+  for (int e = 0; e < 8; ++e) r[e] = (T)(of[e] * inv * wf[e] * gate_f((float)gv[e], silu));
   if (ok) st8<T>(out + row * out_stride + c0, r);
 }
 
@@ -584,8 +587,8 @@ VDAMD_API int vdamd_layer_norm_to(void* out, void* x, long x_stride, const void*
 }
 
 VDAMD_API int vdamd_gated_rms_norm(void* out, long out_stride, const float* o, const float* w, const void* gate,
-                                   long gate_stride, float eps, int rows, int N, int group, float scale, int gate_dt,
-                                   int out_dt, hipStream_t stream) {
+                                   long gate_stride, float eps, int rows, int N, int group, float scale, int silu,
+                                   int gate_dt, int out_dt, hipStream_t stream) {
   if (rows <= 0) return 0;
   if (N <= 0 || group < 0 || (group > 0 && N % group) || out_stride < N) return 1;
   int inner = 0;
@@ -599,7 +602,7 @@ VDAMD_API int vdamd_gated_rms_norm(void* out, long out_stride, const float* o, c
         if constexpr (!std::is_same_v<TG, float>)
           hipLaunchKernelGGL((gated_group_norm_vec_kernel<TG>), dim3((unsigned)((units * L + 255) / 256)), dim3(256), 0,
                              stream, (TG*)out, out_stride, o, w, (const TG*)gate, gate_stride, eps, units, N, group, L,
-                             scale);
+                             scale, silu);
       });
       if (rv) return 1;
       HIP_LAUNCH_CHECK();
@@ -610,14 +613,14 @@ VDAMD_API int vdamd_gated_rms_norm(void* out, long out_stride, const float* o, c
       inner = by_dtype(out_dt, [&](auto* to) {
         using TO = std::remove_pointer_t<decltype(to)>;
         hipLaunchKernelGGL((gated_group_norm_kernel<TG, TO>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, stream,
-                           (TO*)out, out_stride, o, w, (const TG*)gate, gate_stride, eps, rows, N, group, scale);
+                           (TO*)out, out_stride, o, w, (const TG*)gate, gate_stride, eps, rows, N, group, scale, silu);
       });
     });
     if (rc | inner) return 1;
     HIP_LAUNCH_CHECK();
     return 0;
   }
-  if (scale == 1.0f && out_stride == N && gate_dt != DT_F32 && gate_dt == out_dt && N % 8 == 0 && gate_stride % 8 == 0 && aligned16(gate) && aligned16(o) &&
+  if (scale == 1.0f && !silu && out_stride == N && gate_dt != DT_F32 && gate_dt == out_dt && N % 8 == 0 && gate_stride % 8 == 0 && aligned16(gate) && aligned16(o) &&
       aligned16(w) && aligned16(out)) {
     const int rv = by_dtype(gate_dt, [&](auto* tg) {
       using TG = std::remove_pointer_t<decltype(tg)>;
@@ -634,7 +637,7 @@ VDAMD_API int vdamd_gated_rms_norm(void* out, long out_stride, const float* o, c
     inner = by_dtype(out_dt, [&](auto* to) {
       using TO = std::remove_pointer_t<decltype(to)>;
       hipLaunchKernelGGL((gated_rms_norm_kernel<TG, TO>), dim3(rows), dim3(row_threads(N)), 0, stream, (TO*)out,
-                         out_stride, o, w, (const TG*)gate, gate_stride, eps, N, scale);
+                         out_stride, o, w, (const TG*)gate, gate_stride, eps, N, scale, silu);
     });
   });
   if (rc | inner) return 1;

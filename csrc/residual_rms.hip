@@ -3,12 +3,13 @@
 //
 //   residual_rms     one launch per sublayer boundary.  With x the fp32 residual stream (updated in place):
 //                      x += a + b                      (outputs of two sublayers that read the same input; either absent)
-//                      x += y / rms(y) * post_w        (an output that is RMS-normed before it joins the stream; absent)
+//                      x += y / rms(y) * post_w * post_scale (an output RMS-normed before it joins the stream; absent)
 //                      out = x / rms(x) * (offset + w) (the next sublayer's input) or out = x, in any float type
 //                    and, with nothing to add, the plain RMS norm of rows of any float type (fp32 gains)
 //   gelu_mul_rows    gelu_tanh(g[t, :]) * table[ids[t], col : col + n]
 //   sigmoid_mul      o * sigmoid(gate) * scale into a destination with strided rows
 //   gelu             the tanh form or the exact one, element-wise
+//   gelu_and_mul     gelu(x[:, :F]) * x[:, F:]
 #include "common.h"
 #include <math.h>
 #include <type_traits>
@@ -69,6 +70,7 @@ struct ResidualArgs {
   const float* w;                    // [H] or null: no gain
   float offset, eps;
   int H, normed;
+  float post_scale;                  // (with y)
 };
 
 // W values per thread and turn (4: rows whose length, strides and addresses allow 16 / 8-byte accesses).  A row is
@@ -89,7 +91,7 @@ __global__ void residual_rms_kernel(ResidualArgs p) {
       if constexpr (W == 4) { const f32x4 v = ld4<TA>(yr + 4 * i); ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
       else { const float v = ldf(yr + i); ss += v * v; }
     }
-    inv_y = 1.0f / sqrtf(block_sum(ss, red) / (float)p.H + p.eps);
+    inv_y = p.post_scale / sqrtf(block_sum(ss, red) / (float)p.H + p.eps);
   }
   const bool adds = ar != nullptr || yr != nullptr;
   float ss = 0.f;
@@ -189,6 +191,31 @@ __global__ void gelu_kernel(T* __restrict__ out, const T* __restrict__ x, long n
   }
 }
 
+// W values per thread: rows of [g (F) | u (F)]
+template <typename T, int W>
+__global__ void gelu_and_mul_kernel(T* __restrict__ out, const T* __restrict__ x, long x_stride, int F, int rows,
+                                    int tanh_form) {
+  const int per = F / W;
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= (long)rows * per) return;
+  const long t = i / per;
+  const int j = (int)(i - t * per) * W;
+  const T* g = x + t * x_stride + j;
+  if constexpr (W == 8) {
+    const typename Vec8<T>::type gv = ld8<T>(g), uv = ld8<T>(g + F);
+    typename Vec8<T>::type r;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float z = (float)gv[e];
+      r[e] = (T)((tanh_form ? gelu_tanh_f(z) : gelu_erf_f(z)) * (float)uv[e]);
+    }
+    st8<T>(out + t * F + j, r);
+  } else {
+    const float z = ldf(g);
+    stf(out + t * F + j, (tanh_form ? gelu_tanh_f(z) : gelu_erf_f(z)) * ldf(g + F));
+  }
+}
+
 }  // namespace
 
 // x_dt: the type of x (DT_F32 whenever a / b / y is given: x is then the residual stream, updated in place);
@@ -196,11 +223,12 @@ __global__ void gelu_kernel(T* __restrict__ out, const T* __restrict__ x, long n
 VDAMD_API int vdamd_residual_rms(void* out, long out_stride, void* x, long x_stride, const void* a, long a_stride,
                                  const void* b, long b_stride, const void* y, long y_stride, const float* post_w,
                                  const float* w, float offset, float eps, int rows, int H, int normed, int x_dt,
-                                 int in_dt, int out_dt, hipStream_t stream) {
+                                 int in_dt, int out_dt, float post_scale, hipStream_t stream) {
   if (rows <= 0) return 0;
   if (H <= 0 || (b != nullptr && a == nullptr) || (y != nullptr && post_w == nullptr)) return 1;
   if ((a != nullptr || y != nullptr) && x_dt != DT_F32) return 1;
-  ResidualArgs p{out, out_stride, x, x_stride, a, a_stride, b, b_stride, y, y_stride, post_w, w, offset, eps, H, normed};
+  ResidualArgs p{out, out_stride, x, x_stride, a, a_stride, b, b_stride, y, y_stride, post_w, w, offset, eps, H, normed,
+                 post_scale};
   const bool vec = H % 4 == 0 && x_stride % 4 == 0 && out_stride % 4 == 0 && a_stride % 4 == 0 && b_stride % 4 == 0 &&
                    y_stride % 4 == 0 && aligned16(x) && aligned16(out) && aligned16(a) && aligned16(b) &&
                    aligned16(y) && aligned16(w) && aligned16(post_w);
@@ -279,6 +307,33 @@ VDAMD_API int vdamd_gelu(void* out, const void* x, long n, int tanh_form, int dt
       }
     }
     if (!done) hipLaunchKernelGGL((gelu_kernel<TT, 1>), grid, dim3(256), 0, stream, (TT*)out, (const TT*)x, n, tanh_form);
+  });
+  if (rc) return 1;
+  HIP_LAUNCH_CHECK();
+  return 0;
+}
+
+// x [rows, x_stride] = [g (F) | u (F)], out [rows, F] contiguous
+VDAMD_API int vdamd_gelu_and_mul(void* out, const void* x, long x_stride, int rows, int F, int tanh_form, int dt,
+                                 hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (F <= 0) return 1;
+  const bool vec = dt != DT_F32 && F % 8 == 0 && x_stride % 8 == 0 && aligned16(out) && aligned16(x);
+  const long total = (long)rows * (vec ? F / 8 : F);
+  const dim3 grid((unsigned)((total + 255) / 256));
+  const int rc = by_dtype(dt, [&](auto* tp) {
+    using TT = std::remove_pointer_t<decltype(tp)>;
+    bool done = false;
+    if constexpr (!std::is_same_v<TT, float>) {
+      if (vec) {
+        hipLaunchKernelGGL((gelu_and_mul_kernel<TT, 8>), grid, dim3(256), 0, stream, (TT*)out, (const TT*)x, x_stride, F,
+                           rows, tanh_form);
+        done = true;
+      }
+    }
+    if (!done)
+      hipLaunchKernelGGL((gelu_and_mul_kernel<TT, 1>), grid, dim3(256), 0, stream, (TT*)out, (const TT*)x, x_stride, F,
+                         rows, tanh_form);
   });
   if (rc) return 1;
   HIP_LAUNCH_CHECK();

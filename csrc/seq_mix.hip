@@ -11,6 +11,8 @@
 //                          their position, value i paired with value i + half)
 //   short_conv_act         the convolution alone over the leading columns of a fused projection, through SiLU when
 //                          asked, result in the activation type
+//   rotate_norm_cache      q and k heads of a fused projection rotated by their position (cos and sin once per row, in
+//                          LDS) and THEN RMS-normed per head; k and v into the caches, q out
 //   conv_state_update      the last taps-1 projected rows of every sequence into its state slot
 //   window_bias_attention  attention over the caches K [blocks, Hkv, block, D] (key rows) and V [blocks, Hkv,
 //                          block / 8, Dv, 8] (8 keys side by side per channel: the V^T operand of the matrix cores
@@ -501,7 +503,7 @@ __global__ void conv_state_update_kernel(const T* __restrict__ x, long x_stride,
 }
 
 // The convolution alone (no head structure): out[t, c] = act(bias[c] + sum_j w[j, c] * u[t - taps + 1 + j, c]) for the
-// first C columns of x (plus u[t, c] itself with `residual`), history from the step's own rows or the state slot as above.  One thread per (row, channel); the 16-bit
+// first C columns of x (u = the input plus in_bias[c] where the position exists; plus u[t, c] itself with `residual`), history from the step's own rows or the state slot as above.  One thread per (row, channel); the 16-bit
 // variant gives a thread 8 neighbouring channels (16-byte accesses).  A sequence's only row moves its state on here.
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void short_conv_act_kernel(T* __restrict__ out, long out_stride, const T* __restrict__ x,
@@ -510,7 +512,8 @@ __global__ __launch_bounds__(256) void short_conv_act_kernel(T* __restrict__ out
                                                              const int* __restrict__ seq_lens,
                                                              const int* __restrict__ token_seq,
                                                              const int* __restrict__ positions, int C, int taps, int silu,
-                                                             const float* __restrict__ bias, int residual) {
+                                                             const float* __restrict__ bias, int residual,
+                                                             const float* __restrict__ in_bias) {
   constexpr int W = VEC ? 8 : 1;
   const int t = blockIdx.x;
   const int c = (blockIdx.y * blockDim.x + threadIdx.x) * W;
@@ -522,9 +525,9 @@ __global__ __launch_bounds__(256) void short_conv_act_kernel(T* __restrict__ out
   const int R = taps - 1;
   T* st = state + (long)slots[s] * (R > 0 ? R : 1) * C;
   const bool own_state = (n == 1) && R > 0;
-  float acc[W], cur[W];
+  float acc[W], cur[W], ib[W];
 #pragma unroll
-  for (int e = 0; e < W; ++e) { acc[e] = bias ? bias[c + e] : 0.f; cur[e] = 0.f; }
+  for (int e = 0; e < W; ++e) { acc[e] = bias ? bias[c + e] : 0.f; cur[e] = 0.f; ib[e] = in_bias ? in_bias[c + e] : 0.f; }
   for (int j = 0; j < taps; ++j) {
     const int back = taps - 1 - j;
     const int p = pos - back;
@@ -540,13 +543,13 @@ __global__ __launch_bounds__(256) void short_conv_act_kernel(T* __restrict__ out
       }
       if (own_state && j >= 1) st8<T>(st + (long)(j - 1) * C + c, u);       // (row j - 1 was read one turn earlier)
 #pragma unroll
-      for (int e = 0; e < 8; ++e) { acc[e] += (float)wv[e] * (float)u[e]; cur[e] = (float)u[e]; }
+      for (int e = 0; e < 8; ++e) { acc[e] += (float)wv[e] * ((float)u[e] + (p >= 0 ? ib[e] : 0.f)); cur[e] = (float)u[e]; }
     } else {
       float u = 0.f;
       if (p >= chunk_start && p >= 0) u = ldf(x + (long)(t - back) * x_stride + c);
       else if (p >= 0) u = ldf(st + (long)(R - (chunk_start - p)) * C + c);
       if (own_state && j >= 1) stf(st + (long)(j - 1) * C + c, u);
-      acc[0] += ldf(w + (long)j * C + c) * u;
+      acc[0] += ldf(w + (long)j * C + c) * (u + (p >= 0 ? ib[0] : 0.f));
       cur[0] = u;
     }
   }
@@ -565,6 +568,130 @@ __global__ __launch_bounds__(256) void short_conv_act_kernel(T* __restrict__ out
     st8<T>(out + (long)t * out_stride + c, o);
   } else {
     stf(out + (long)t * out_stride + c, acc[0]);
+  }
+}
+
+// ---------------------------------------------------------------------------- rotation, head norm, cache write
+struct RotArgs {
+  const void* x; long x_stride;             // [T, x_stride]: [q | k | v | ...]
+  const float* inv_freq; int half;          // [half] angular frequencies
+  float rot_scale, eps;                     // factor on cos and sin
+  const float* q_norm; const float* k_norm; // [D] or null
+  const int* positions;                     // [T]
+  void* q_out;                              // [T, H, D]
+  void* k_cache; void* v_cache;             // [blocks, G, bs, D], [blocks, G, bs / 8, Dv, 8] or null
+  const int* slot_mapping;                  // [T]
+  int H, G, D, Dv, bs, interleaved;
+};
+
+constexpr int ROT_MAX_HALF = 256;
+
+__device__ __forceinline__ void rot_table(const RotArgs& a, int pos, float* cs, float* sn) {
+  for (int i = threadIdx.x; i < a.half; i += blockDim.x) {
+    const float ang = (float)pos * a.inv_freq[i];
+    cs[i] = cosf(ang) * a.rot_scale;
+    sn[i] = sinf(ang) * a.rot_scale;
+  }
+  __syncthreads();
+}
+
+// grid (rows): a wave per head in turn, any head size up to 512, either pairing
+template <typename T>
+__global__ __launch_bounds__(256) void rotate_norm_cache_kernel(RotArgs a) {
+  __shared__ float cs[ROT_MAX_HALF], sn[ROT_MAX_HALF];
+  const long t = blockIdx.x;
+  rot_table(a, a.positions[t], cs, sn);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nwaves = blockDim.x >> 6;
+  const T* xr = (const T*)a.x + t * a.x_stride;
+  const int slot = a.k_cache != nullptr ? a.slot_mapping[t] : -1;
+  const long blk = slot >= 0 ? slot / a.bs : 0;
+  const int off = slot >= 0 ? slot % a.bs : 0;
+  for (int u = wave; u < a.H + a.G; u += nwaves) {
+    const T* src = xr + (long)u * a.D;
+    float v[UNIT_MAX_PER_LANE];
+    float ss = 0.f;
+#pragma unroll
+    for (int it = 0; it < UNIT_MAX_PER_LANE; ++it) {
+      const int d = lane + it * 64;
+      v[it] = 0.f;
+      if (d >= a.D) continue;
+      v[it] = ldf(src + d);
+      if (d < 2 * a.half) {
+        const int i = a.interleaved ? d >> 1 : (d < a.half ? d : d - a.half);
+        const bool second = a.interleaved ? (d & 1) : d >= a.half;
+        const int pd = a.interleaved ? d ^ 1 : (second ? d - a.half : d + a.half);
+        const float o = ldf(src + pd);
+        v[it] = second ? v[it] * cs[i] + o * sn[i] : v[it] * cs[i] - o * sn[i];
+      }
+      ss += v[it] * v[it];
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.D + a.eps);
+    const bool is_q = u < a.H;
+    const float* w = is_q ? a.q_norm : a.k_norm;
+    if (!is_q && slot < 0) continue;
+    T* dst = is_q ? (T*)a.q_out + (t * a.H + u) * (long)a.D
+                  : (T*)a.k_cache + ((blk * a.G + (u - a.H)) * a.bs + off) * (long)a.D;
+#pragma unroll
+    for (int it = 0; it < UNIT_MAX_PER_LANE; ++it) {
+      const int d = lane + it * 64;
+      if (d < a.D) stf(dst + d, v[it] * inv * (w ? w[d] : 1.f));
+    }
+  }
+  if (slot < 0) return;
+  const T* vr = xr + (long)(a.H + a.G) * a.D;
+  for (int i = threadIdx.x; i < a.G * a.Dv; i += blockDim.x) {
+    const int g = i / a.Dv, d = i - g * a.Dv;
+    ((T*)a.v_cache)[(((blk * a.G + g) * (a.bs >> 3) + (off >> 3)) * (long)a.Dv + d) * 8 + (off & 7)] = vr[i];
+  }
+}
+
+// 16-bit types, neighbouring pairs, head sizes of 8 L with L a power of two: a lane owns 8 channels (4 pairs) of a head,
+// the sum of squares over the head's L neighbouring lanes by xor-shuffles
+template <typename T>
+__global__ __launch_bounds__(256) void rotate_norm_cache_vec_kernel(RotArgs a, int L) {
+  using V8 = typename Vec8<T>::type;
+  __shared__ float cs[ROT_MAX_HALF], sn[ROT_MAX_HALF];
+  const long t = blockIdx.x;
+  rot_table(a, a.positions[t], cs, sn);
+  const T* xr = (const T*)a.x + t * a.x_stride;
+  const int slot = a.k_cache != nullptr ? a.slot_mapping[t] : -1;
+  const long blk = slot >= 0 ? slot / a.bs : 0;
+  const int off = slot >= 0 ? slot % a.bs : 0;
+  const int sh = __builtin_ctz(L);
+  // (the lanes of a head enter a turn of the loop together: L divides the wave and the stride)
+  for (int idx = threadIdx.x; idx < (a.H + a.G) * L; idx += blockDim.x) {
+    const int u = idx >> sh, d = (idx & (L - 1)) * 8;
+    const V8 xv = ld8<T>(xr + (long)u * a.D + d);
+    float v[8];
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; e += 2) {
+      const int i = (d + e) >> 1;
+      const float p = (float)xv[e], q = (float)xv[e + 1];
+      const bool rot = i < a.half;
+      const float c = rot ? cs[i] : 1.f, s = rot ? sn[i] : 0.f;
+      v[e] = p * c - q * s;
+      v[e + 1] = q * c + p * s;
+      ss += v[e] * v[e] + v[e + 1] * v[e + 1];
+    }
+    for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
+    const float inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+    const bool is_q = u < a.H;
+    const float* w = is_q ? a.q_norm : a.k_norm;
+    V8 r;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) r[e] = (T)(v[e] * inv * (w ? w[d + e] : 1.f));
+    if (is_q) st8<T>((T*)a.q_out + (t * a.H + u) * (long)a.D + d, r);
+    else if (slot >= 0) st8<T>((T*)a.k_cache + ((blk * a.G + (u - a.H)) * a.bs + off) * (long)a.D + d, r);
+  }
+  if (slot < 0) return;
+  const T* vr = xr + (long)(a.H + a.G) * a.D;
+  for (int i = threadIdx.x * 8; i < a.G * a.Dv; i += blockDim.x * 8) {
+    const int g = i / a.Dv, d = i - g * a.Dv;                     // (Dv % 8 == 0: the 8 channels share a head)
+    const V8 vv = ld8<T>(vr + i);
+    T* vd = (T*)a.v_cache + (((blk * a.G + g) * (a.bs >> 3) + (off >> 3)) * (long)a.Dv + d) * 8 + (off & 7);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) vd[e * 8] = vv[e];
   }
 }
 
@@ -1147,12 +1274,45 @@ VDAMD_API int vdamd_conv_norm_cache(const void* x, long x_stride, const void* co
   });
 }
 
+// x [T, x_stride] = [q (H * D) | k (G * D) | v (G * Dv)], q_out [T, H, D]; caches may be null (nothing is written then).
+// inv_freq [half] (null with half 0), 2 half <= D <= 512; interleaved: neighbours are paired, else values half apart
+VDAMD_API int vdamd_rotate_norm_cache(void* q_out, const void* x, long x_stride, const float* inv_freq, int half,
+                                      float rot_scale, int interleaved, float eps, const float* q_norm,
+                                      const float* k_norm, const int* positions, void* k_cache, void* v_cache,
+                                      const int* slot_mapping, int T, int H, int G, int D, int Dv, int bs, int dt,
+                                      hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (H <= 0 || G <= 0 || H % G || D <= 0 || D > 64 * UNIT_MAX_PER_LANE || Dv <= 0 || half < 0 || 2 * half > D ||
+      half > ROT_MAX_HALF || (half > 0 && inv_freq == nullptr))
+    return 1;
+  if (k_cache != nullptr && (v_cache == nullptr || slot_mapping == nullptr || bs <= 0 || bs % 8)) return 1;
+  RotArgs a{x, x_stride, inv_freq, half, rot_scale, eps, q_norm, k_norm, positions, q_out, k_cache, v_cache, slot_mapping,
+            H, G, D, Dv, bs, interleaved};
+  const int L = D / 8;
+  auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = dt != DT_F32 && (interleaved || half == 0) && D % 8 == 0 && (L & (L - 1)) == 0 && L <= 64 &&
+                   Dv % 8 == 0 && x_stride % 8 == 0 && al16(x) && al16(q_out) && al16(k_cache);
+  return by_dtype(dt, [&](auto* tp) {
+    using TT = std::remove_pointer_t<decltype(tp)>;
+    if constexpr (!std::is_same_v<TT, float>) {
+      if (vec) {
+        const int lanes = (H + G) * L;
+        hipLaunchKernelGGL((rotate_norm_cache_vec_kernel<TT>), dim3(T), dim3(lanes >= 256 ? 256 : (lanes >= 128 ? 128 : 64)),
+                           0, stream, a, L);
+        return;
+      }
+    }
+    hipLaunchKernelGGL((rotate_norm_cache_kernel<TT>), dim3(T), dim3(256), 0, stream, a);
+  });
+}
+
 // out [T, out_stride] = act(conv over time of x[:, :C]); state [slots, max(taps - 1, 1), C] moves on.  update_multi: 0
 // when every sequence of the step has one row
 VDAMD_API int vdamd_short_conv_act(void* out, long out_stride, const void* x, long x_stride, const void* conv_w,
                                    void* state, const int* slots, const int* qsl, const int* seq_lens,
                                    const int* token_seq, const int* positions, int T, int B, int C, int taps, int silu,
-                                   int update_multi, const float* bias, int residual, int dt, hipStream_t stream) {
+                                   int update_multi, const float* bias, int residual, const float* in_bias, int dt,
+                                   hipStream_t stream) {
   if (T <= 0) return 0;
   if (taps < 1 || taps > CONV_MAX_TAPS || C <= 0) return 1;
   const int R = taps - 1;
@@ -1165,14 +1325,14 @@ VDAMD_API int vdamd_short_conv_act(void* out, long out_stride, const void* x, lo
       if (vec) {
         hipLaunchKernelGGL((short_conv_act_kernel<TT, true>), dim3(T, (C / 8 + 255) / 256), dim3(256), 0, stream,
                            (TT*)out, out_stride, (const TT*)x, x_stride, (const TT*)conv_w, (TT*)state, slots, qsl,
-                           seq_lens, token_seq, positions, C, taps, silu, bias, residual);
+                           seq_lens, token_seq, positions, C, taps, silu, bias, residual, in_bias);
         done = true;
       }
     }
     if (!done)
       hipLaunchKernelGGL((short_conv_act_kernel<TT, false>), dim3(T, (C + 255) / 256), dim3(256), 0, stream, (TT*)out,
                          out_stride, (const TT*)x, x_stride, (const TT*)conv_w, (TT*)state, slots, qsl, seq_lens,
-                         token_seq, positions, C, taps, silu, bias, residual);
+                         token_seq, positions, C, taps, silu, bias, residual, in_bias);
     if (update_multi && R > 0)
       hipLaunchKernelGGL((conv_state_update_kernel<TT>), dim3((C + 255) / 256, B), dim3(256), 0, stream,
                          (const TT*)x, x_stride, (TT*)state, slots, qsl, C, R);

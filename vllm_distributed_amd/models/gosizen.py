@@ -43,6 +43,7 @@ from .layers.attention import (Attention, ResidualRMSNorm, RowLatentAttention, W
 from .layers.linear import ColumnParallelLinear, ReplicatedLinear, RowParallelLinear, VocabParallelEmbedding
 from .layers.linear_attention import DeltaRuleMixer
 from .layers.moe import BiasedTopKMoE
+from .layers.parallel_heads import ParallelHeads
 from .layers.short_conv import ShortConv, SlotState
 from .utils import IntermediateTensors, materialize
 
@@ -169,10 +170,9 @@ class ChunkedConvAttention(nn.Module):
         ops.sigmoid_mul(attn.forward_cached(q), x[:, self.channels:], self.out_scale, out=out)
 
 
-class ParallelMixer(nn.Module):
+class ParallelMixer(ParallelHeads):
     def __init__(self, width: int, m: dict, eps: float, layer_idx: int, dtype: torch.dtype, passes: int,
                  shapes: Dict[str, Tuple[int, ...]]):
-        super().__init__()
         right = dict(m["right"])
         # the widths of the two low-rank projections are sizes only the tensors state
         for key, tensor in (("decay_rank", "a1"), ("gate_rank", "g1")):
@@ -182,17 +182,10 @@ class ParallelMixer(nn.Module):
                     raise ValueError(f"layer {layer_idx}: neither the config ({key}) nor a checkpoint tensor "
                                      f"(mix.right.{tensor}) gives the width of the low-rank projection")
                 right[key] = int(shape[0])
-        self.left = ChunkedConvAttention(width, m["left"], eps, layer_idx, dtype, passes, float(m.get("left_scale", 1.0)))
-        self.right = DeltaRuleMixer(width, right, eps, layer_idx, dtype, passes, float(m.get("right_scale", 1.0)))
-        self.dtype = dtype
-        self.o = RowParallelLinear(self.left.out_cols + self.right.out_cols, width, False, dtype)
-
-    def forward(self, h: torch.Tensor, index: int) -> torch.Tensor:
-        nl = self.left.out_cols
-        heads = torch.empty((h.shape[0], nl + self.right.out_cols), dtype=self.dtype, device=h.device)
-        self.left(h, index, heads[:, :nl])
-        self.right(h, index, heads[:, nl:])
-        return self.o(heads)
+        super().__init__(ChunkedConvAttention(width, m["left"], eps, layer_idx, dtype, passes,
+                                              float(m.get("left_scale", 1.0))),
+                         DeltaRuleMixer(width, right, eps, layer_idx, dtype, passes, float(m.get("right_scale", 1.0))),
+                         width, dtype)
 
 
 # ---------------------------------------------------------------------------------------------------- feed-forwards
@@ -429,10 +422,7 @@ class GosizenForCausalLM(nn.Module):
                 continue
             p, shard = params[t[0]], t[1]
             if isinstance(shard, tuple):          # a run of columns of the fused output projection
-                mix = self.layers[int(name[1:].partition(".")[0])].mix
-                lo = 0 if shard[1] == 0 else mix.left.out_cols
-                w = materialize(w)
-                p.data[:, lo:lo + w.shape[1]].copy_(w)
+                self.layers[int(name[1:].partition(".")[0])].mix.load_output_half(shard[1], materialize(w))
                 loaded.append(name)
                 continue
             loader = getattr(p, "weight_loader", None)

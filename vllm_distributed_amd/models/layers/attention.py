@@ -338,7 +338,8 @@ class WindowBiasAttention(Attention):
     first); scores, softmax and the weighted sum of values are fp32 in every dtype.  ``chunk > 0`` replaces the window
     by blocks of ``chunk`` positions counted from the sequence's start: a query sees the keys of its own block up to
     itself (``window`` is then ``chunk``: no key further back is ever read, so the pages behind it are given back).
-    ``sink`` may be another instance's parameter (layers that run several times over one set of weights)."""
+    ``sink`` may be another instance's parameter (layers that run several times over one set of weights), or a float: a
+    fixed score for every head (0.0: one is added to the denominator)."""
     row_cache = True
 
     def __init__(self, num_heads: int, dim: int, vdim: int, num_kv_heads: int, scale: float, layer_idx: int,
@@ -356,6 +357,8 @@ class WindowBiasAttention(Attention):
         self.bias_rate = nn.Parameter(torch.zeros(num_heads, dtype=f32), requires_grad=False) if distance_bias else None
         if isinstance(sink, nn.Parameter):
             self.sink = sink
+        elif isinstance(sink, float):
+            self.register_buffer("sink", torch.full((num_heads,), sink, dtype=f32), persistent=False)
         else:
             self.sink = nn.Parameter(torch.zeros(num_heads, dtype=f32), requires_grad=False) if sink else None
 
@@ -453,7 +456,8 @@ class ResidualRMSNorm(nn.Module):
     """RMS norm over an fp32 residual stream in fp32 arithmetic, with fp32 gains ``offset + weight`` (``offset`` 1: the
     checkpoint keeps the gain minus one).  ``forward`` returns the model dtype (the input of a projection); ``add`` folds one or
     two sublayer outputs into the stream and hands back the normed sum in the same launch; ``after`` does so for an
-    output that is itself RMS-normed with ``post_weight`` before it joins the stream."""
+    output that is itself RMS-normed with ``post_weight`` before it joins the stream, ``fold`` for an output that THIS
+    norm is for."""
 
     def __init__(self, hidden_size: int, eps: float, dtype: torch.dtype, offset: float = 0.0):
         super().__init__()
@@ -468,6 +472,15 @@ class ResidualRMSNorm(nn.Module):
 
     def after(self, y: torch.Tensor, post_weight: torch.Tensor, residual: torch.Tensor) -> torch.Tensor:
         return ops.norm_add_norm(y, post_weight, residual, self.weight, self.eps, self.dtype, self.offset)
+
+    def fold(self, y: torch.Tensor, residual: torch.Tensor, scale: float = 1.0,
+             then: Optional["ResidualRMSNorm"] = None) -> torch.Tensor:
+        """This norm as a sublayer's OUTPUT norm: ``residual += scale * norm(y)``; returns ``then(residual)``, or with
+        ``then`` None the stream itself in the model dtype (the next sublayer reads it un-normed).  One launch."""
+        if self.offset:
+            raise NotImplementedError("an output norm's gain is stored whole")
+        return ops.norm_add_norm(y, self.weight, residual, None if then is None else then.weight, self.eps, self.dtype,
+                                 0.0 if then is None else then.offset, then is not None, scale)
 
 
 class RMSNorm(nn.Module):

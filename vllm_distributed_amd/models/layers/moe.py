@@ -598,11 +598,13 @@ class BiasedTopKMoE(FusedMoE):
 
 
 class GatedMLP(nn.Module):
-    """One feed-forward of the gated form ``down(silu(gate(x)) * up(x))``, gate and up as one fused projection; no
-    biases.  The inner width is zero-padded to a multiple of 8 (the activation kernel's 16-byte accesses)."""
+    """One feed-forward of the gated form ``down(act(gate(x)) * up(x))`` (``activation``: SiLU, or a GELU by its name),
+    gate and up as one fused projection; no biases.  The inner width is zero-padded to a multiple of 8 (the activation
+    kernels' 16-byte accesses)."""
 
-    def __init__(self, hidden: int, inter: int, dtype: torch.dtype):
+    def __init__(self, hidden: int, inter: int, dtype: torch.dtype, activation: str = "silu"):
         super().__init__()
+        self.activation = activation
         self.inter, self.i_pad = inter, (inter + 7) // 8 * 8
         self.w13 = nn.Parameter(torch.zeros(2 * self.i_pad, hidden, dtype=dtype), requires_grad=False)
         self.w2 = nn.Parameter(torch.zeros(hidden, self.i_pad, dtype=dtype), requires_grad=False)
@@ -619,7 +621,7 @@ class GatedMLP(nn.Module):
         param.data[:, :self.inter].copy_(materialize(w))
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
-        return ops.linear(ops.silu_and_mul(ops.linear(x, self.w13)), self.w2)
+        return ops.linear(ops.act_and_mul(ops.linear(x, self.w13), self.activation), self.w2)
 
 
 class ScoredTopKMoE(FusedMoE):

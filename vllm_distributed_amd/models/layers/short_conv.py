@@ -9,7 +9,7 @@ because of where they are, not because of what the slot holds.
 """
 from __future__ import annotations
 
-from typing import Optional, Sequence, Tuple
+from typing import Dict, Optional, Sequence, Tuple
 
 import torch
 import torch.nn as nn
@@ -58,6 +58,18 @@ class ShortConv(nn.Module):
 
     def bind_state(self, state: Optional[torch.Tensor]) -> None:
         self.state = state
+
+
+def stated_taps(shapes: Dict[str, Tuple[int, ...]], tensor: str, stated) -> int:
+    """Taps of a convolution: the checkpoint tensor's second dimension where there is one, else what the config
+    states."""
+    shape = shapes.get(tensor)
+    return int(shape[1]) if shape is not None and len(shape) == 2 else int(stated or 0)
+
+
+def conv_rows(md, positions: torch.Tensor) -> Optional[torch.Tensor]:
+    """The sequence of every row of the step (None in a pure decode batch: row ``t`` is sequence ``t``)."""
+    return None if md.num_prefills == 0 else md.token_rows(positions)[0]
 
 
 class SlotState:

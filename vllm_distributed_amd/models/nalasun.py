@@ -40,24 +40,12 @@ from .layers.attention import Attention, CrossedBiasAttention, ResidualRMSNorm, 
 from .layers.linear import ColumnParallelLinear, RowParallelLinear, VocabParallelEmbedding
 from .layers.linear_attention import DeltaRuleMixer, SelectiveStateSpace
 from .layers.moe import ScoredTopKMoE
-from .layers.short_conv import ShortConv, SlotState
+from .layers.short_conv import ShortConv, SlotState, conv_rows, stated_taps
 from .utils import IntermediateTensors, materialize
 
 
 def _f32(*shape: int) -> nn.Parameter:
     return nn.Parameter(torch.zeros(shape, dtype=torch.float32), requires_grad=False)
-
-
-def _taps(shapes: Dict[str, Tuple[int, ...]], tensor: str, stated) -> int:
-    """Taps of a convolution: the checkpoint tensor's second dimension where there is one, else what the config
-    states."""
-    shape = shapes.get(tensor)
-    return int(shape[1]) if shape is not None and len(shape) == 2 else int(stated or 0)
-
-
-def _conv_rows(md, positions):
-    """The sequence of every row of the step (None in a pure decode batch: row ``t`` is sequence ``t``)."""
-    return None if md.num_prefills == 0 else md.token_rows(positions)[0]
 
 
 # ---------------------------------------------------------------------------------------------------- mixers
@@ -109,7 +97,7 @@ class ChannelDeltaMixer(nn.Module):
                     raise ValueError(f"layer {layer_idx}: neither the config ({key}) nor a checkpoint tensor "
                                      f"(mix.{tensor}) gives the width of the low-rank projection")
                 m[key] = int(shape[0])
-        m["conv"] = _taps(shapes, f"l{layer_idx}.mix.q.conv", m.get("conv")) or 1
+        m["conv"] = stated_taps(shapes, f"l{layer_idx}.mix.q.conv", m.get("conv")) or 1
         self.dtype = dtype
         self.inner = DeltaRuleMixer(width, m, eps, layer_idx, dtype, 1, 1.0)
         self.o = RowParallelLinear(self.inner.out_cols, width, False, dtype)
@@ -137,7 +125,7 @@ class StateSpaceMixer(nn.Module):
         bc = groups * n
         # [z | x | B | C | dt]
         self.proj = ColumnParallelLinear(width, [self.inner_cols, self.inner_cols, bc, bc, heads], False, dtype)
-        self.conv = ShortConv([self.inner_cols, bc, bc], _taps(shapes, f"l{layer_idx}.mix.conv", m.get("conv")) or 1,
+        self.conv = ShortConv([self.inner_cols, bc, bc], stated_taps(shapes, f"l{layer_idx}.mix.conv", m.get("conv")) or 1,
                               dtype, bias=True)
         self.conv_state = SlotState((max(self.conv.taps - 1, 1), self.conv.channels))
         self.ssm_state = SlotState(self.ssm.per_slot_shape(), torch.float32)
@@ -156,7 +144,7 @@ class StateSpaceMixer(nn.Module):
         c = self.conv.channels
         lo = self.inner_cols
         xbc = ops.short_conv_act(u[:, lo:], c, self.conv.weight_t, self.conv_state.state, md.state_slots,
-                                 md.query_start_loc, md.seq_lens, _conv_rows(md, ctx.positions), ctx.positions, True,
+                                 md.query_start_loc, md.seq_lens, conv_rows(md, ctx.positions), ctx.positions, True,
                                  md.num_prefills > 0, self.conv.bias)
         y = self.ssm(xbc, u[:, lo + c:], self.ssm_state.state)
         return self.o(ops.act_gate_group_norm(y, u[:, :lo], self.norm, self.eps, self.norm_group, self.dtype))
@@ -209,7 +197,7 @@ class NalasunLayer(nn.Module):
         md = ctx.attn_metadata
         if self.canon is not None and md is not None:
             h = ops.short_conv_act(h, self.width, self.canon.weight_t, self.canon_state.state, md.state_slots,
-                                   md.query_start_loc, md.seq_lens, _conv_rows(md, ctx.positions), ctx.positions,
+                                   md.query_start_loc, md.seq_lens, conv_rows(md, ctx.positions), ctx.positions,
                                    False, md.num_prefills > 0, None, True)
         y = self.mix(h)
         if self.mlp is None:
@@ -241,7 +229,7 @@ class NalasunForCausalLM(nn.Module):
         from ..config import resolve_model_path
         from .loader import checkpoint_tensor_shapes
         shapes = {} if mc.load_format == "dummy" else checkpoint_tensor_shapes(resolve_model_path(mc.model))
-        taps = _taps(shapes, "l0.canon1", (cfg.get("canon") or {}).get("taps"))
+        taps = stated_taps(shapes, "l0.canon1", (cfg.get("canon") or {}).get("taps"))
         positions = int(cfg.get("max_positions") or (shapes.get("pos") or (0,))[0])
         if positions <= 0:
             raise ValueError("neither the config (max_positions) nor a checkpoint tensor (pos) gives the number of positions")

@@ -80,6 +80,10 @@ _MODELS: Dict[str, Tuple[str, str]] = {
     # weighted by sigmoid scores
     "NalasunForCausalLM": ("nalasun", "NalasunForCausalLM"),
     "Nalasun": ("nalasun", "NalasunForCausalLM"),
+    # fp32 residual stream read un-normed, norms on the sublayers' outputs; a gated linear unit recurrence, a selective
+    # scan per channel, attention over rotated-then-normed heads beside the gated delta rule
+    "KefuraxForCausalLM": ("kefurax", "KefuraxForCausalLM"),
+    "Kefurax": ("kefurax", "KefuraxForCausalLM"),
     # draft heads of speculative decoding (never a served model by themselves; worker/draft_model.py)
     "EagleLlamaForCausalLM": ("spec_heads", "EagleLlamaForCausalLM"),
     "Eagle3LlamaForCausalLM": ("spec_heads", "Eagle3LlamaForCausalLM"),
@@ -92,7 +96,7 @@ _MODELS: Dict[str, Tuple[str, str]] = {
 # architectures whose layers keep per-request state besides the KV cache (convolution tails, recurrences): a cached
 # prefix's blocks do not bring that state back, so prefix reuse is off for them
 _KEEPS_REQUEST_STATE = {"TavulixForCausalLM", "Tavulix", "KabapelForCausalLM", "Kabapel", "GosizenForCausalLM",
-                        "Gosizen", "NalasunForCausalLM", "Nalasun"}
+                        "Gosizen", "NalasunForCausalLM", "Nalasun", "KefuraxForCausalLM", "Kefurax"}
 
 
 def keeps_request_state(arch: str) -> bool:

@@ -291,6 +291,8 @@ def act_and_mul(x, kind: str):
     """``act(x[..., :F]) * x[..., F:]`` for a gated MLP with an activation other than SiLU (GeGLU)."""
     if kind in ("silu", "swish"):
         return silu_and_mul(x)
+    if kind in _GELU_KINDS:
+        return gelu_and_mul(x, _GELU_KINDS[kind] == "tanh")
     f = x.shape[-1] // 2
     return activation(x[..., :f], kind) * x[..., f:]
 
@@ -721,12 +723,14 @@ def decay_linear_attention(x, num_heads: int, dim: int, vdim: int, decay, state,
     return torch_ref.decay_linear_attention(x, num_heads, dim, vdim, decay, state, slots, query_start_loc, seq_lens, silu)
 
 
-def gated_rms_norm(o, weight, gate, eps: float, out_dtype, group: int = 0, scale: float = 1.0, out=None):
+def gated_rms_norm(o, weight, gate, eps: float, out_dtype, group: int = 0, scale: float = 1.0, out=None,
+                   silu: bool = False):
     """RMS norm of fp32 rows (whole rows, or runs of ``group`` values sharing ``weight[group]``) times
-    ``sigmoid(gate) * scale``; ``out``: a view with strided rows that receives the result."""
+    ``sigmoid(gate) * scale`` (``silu``: ``silu(gate) * scale``); ``out``: a view with strided rows that receives the
+    result."""
     if _use_hip(o):
-        return _hip.gated_rms_norm(o, weight, gate, eps, out_dtype, group, scale, out)
-    return torch_ref.gated_rms_norm(o, weight, gate, eps, out_dtype, group, scale, out)
+        return _hip.gated_rms_norm(o, weight, gate, eps, out_dtype, group, scale, out, silu)
+    return torch_ref.gated_rms_norm(o, weight, gate, eps, out_dtype, group, scale, out, silu)
 
 
 def clamped_glu(h, limit: float, alpha: float):
@@ -786,12 +790,14 @@ def add_rms_norm_to(residual, a, b, weight, eps: float, out_dtype, offset: float
 
 
 def norm_add_norm(y, post_weight, residual, next_weight, eps: float, out_dtype, next_offset: float = 0.0,
-                  next_normed: bool = True):
-    """``residual += rms_norm(y) * post_weight`` on the fp32 residual stream and the RMS norm of the sum (or the sum
-    itself) in ``out_dtype``: one launch."""
+                  next_normed: bool = True, post_scale: float = 1.0):
+    """``residual += post_scale * rms_norm(y) * post_weight`` on the fp32 residual stream and the RMS norm of the sum
+    (or the sum itself) in ``out_dtype``: one launch."""
     if _use_hip(y):
-        return _hip.norm_add_norm(y, post_weight, residual, next_weight, eps, out_dtype, next_offset, next_normed)
-    return torch_ref.norm_add_norm(y, post_weight, residual, next_weight, eps, out_dtype, next_offset, next_normed)
+        return _hip.norm_add_norm(y, post_weight, residual, next_weight, eps, out_dtype, next_offset, next_normed,
+                                  post_scale)
+    return torch_ref.norm_add_norm(y, post_weight, residual, next_weight, eps, out_dtype, next_offset, next_normed,
+                                   post_scale)
 
 
 def gelu_mul_rows(g, table, ids, col: int):
@@ -814,21 +820,24 @@ def gelu(x, tanh: bool):
 
 
 def short_conv_act(x, channels: int, conv_weight, state, slots, query_start_loc, seq_lens, token_seq, positions,
-                   silu: bool, has_prefill: bool = True, bias=None, residual: bool = False):
+                   silu: bool, has_prefill: bool = True, bias=None, residual: bool = False, in_bias=None):
     """Causal convolution over time (tap-major ``conv_weight[taps, channels]``, per-request state) of the first
-    ``channels`` columns of a fused projection, plus ``bias``, through SiLU when asked, plus the input itself with
-    ``residual``; see ``torch_ref.short_conv_act``."""
+    ``channels`` columns of a fused projection (``in_bias``: the projection's own bias, added to every input that
+    exists), plus ``bias``, through SiLU when asked, plus the input itself with ``residual``; see
+    ``torch_ref.short_conv_act``."""
+    if residual and in_bias is not None:
+        raise NotImplementedError("the residual form adds the input as it is stored, without its bias")
     if _use_hip(x):
         return _hip.short_conv_act(x, channels, conv_weight, state, slots, query_start_loc, seq_lens, token_seq,
-                                   positions, silu, has_prefill, bias, residual)
+                                   positions, silu, has_prefill, bias, residual, in_bias)
     return torch_ref.short_conv_act(x, channels, conv_weight, state, slots, query_start_loc, seq_lens, silu, bias,
-                                    residual)
+                                    residual, in_bias)
 
 
 def gated_delta_rule(x, num_heads: int, num_qk_heads: int, dim: int, vdim: int, beta, dt, dt_bias, a_log, state,
                      slots, query_start_loc, seq_lens, norm_eps: float = 1e-6, max_query_len: int = 0):
-    """The gated delta rule with a decay per head and key channel and a per-request fp32 state; see
-    ``torch_ref.gated_delta_rule``."""
+    """The gated delta rule with a decay per head and key channel (or, ``dt[T, H]``, per head) and a per-request fp32
+    state; see ``torch_ref.gated_delta_rule``."""
     if _use_hip(x):
         return _hip.gated_delta_rule(x, num_heads, num_qk_heads, dim, vdim, beta, dt, dt_bias, a_log, state, slots,
                                      query_start_loc, seq_lens, norm_eps, max_query_len)
@@ -890,3 +899,46 @@ def mix_heads(o, talk, out_dtype):
     if _use_hip(o):
         return _hip.mix_heads(o, talk, out_dtype)
     return torch_ref.mix_heads(o, talk, out_dtype)
+
+
+# ------------------------------------------------ rotation in front of a head norm, a selective scan per channel, a
+# ------------------------------------------------ gated linear unit recurrence
+def rotate_norm_cache(x, num_heads: int, num_kv_heads: int, dim: int, vdim: int, inv_freq, rot_scale: float,
+                      interleaved: bool, eps: float, q_norm, k_norm, positions, k_cache, v_cache, slot_mapping):
+    """q and k heads rotated, then normed, k and v into the row caches; see ``torch_ref.rotate_norm_cache``."""
+    if _use_hip(x):
+        return _hip.rotate_norm_cache(x, num_heads, num_kv_heads, dim, vdim, inv_freq, rot_scale, interleaved, eps,
+                                      q_norm, k_norm, positions, k_cache, v_cache, slot_mapping)
+    return torch_ref.rotate_norm_cache(x, num_heads, num_kv_heads, dim, vdim, inv_freq, rot_scale, interleaved, eps,
+                                       q_norm, k_norm, positions, k_cache, v_cache, slot_mapping)
+
+
+def gelu_and_mul(x, tanh: bool = True):
+    """``gelu(x[..., :F]) * x[..., F:]`` (the tanh form or the exact one) in fp32 arithmetic, in ``x``'s dtype."""
+    if _use_hip(x):
+        return _hip.gelu_and_mul(x, tanh)
+    return torch_ref.gelu_and_mul(x, tanh)
+
+
+def channel_scan(u, dt, bc, n_state: int, a_log, dt_bias, d_skip, gate, state, slots, query_start_loc, seq_lens,
+                 max_query_len: int = 0):
+    """A selective scan with a state vector and decays per channel and a per-request fp32 state, its output times
+    ``silu(gate)``; see ``torch_ref.channel_scan``.  ``max_query_len`` (0: unknown) only helps the kernel choose its
+    launch."""
+    if _use_hip(u):
+        return _hip.channel_scan(u, dt, bc, n_state, a_log, dt_bias, d_skip, gate, state, slots, query_start_loc,
+                                 seq_lens, max_query_len)
+    return torch_ref.channel_scan(u, dt, bc, n_state, a_log, dt_bias, d_skip, gate, state, slots, query_start_loc,
+                                  seq_lens)
+
+
+def gated_unit_step(u, ra, ra_bias, ri, ri_bias, rate, gate, gate_bias, state, slots, query_start_loc, seq_lens,
+                    max_query_len: int = 0):
+    """Block-diagonal gates, the gated linear unit recurrence with its per-request fp32 state, and its output gate; see
+    ``torch_ref.block_gates`` and ``torch_ref.gated_unit_scan``.  ``max_query_len`` 1: every row is a sequence's only
+    one (a single launch); 0: unknown."""
+    if _use_hip(u):
+        return _hip.gated_unit_step(u, ra, ra_bias, ri, ri_bias, rate, gate, gate_bias, state, slots, query_start_loc,
+                                    seq_lens, max_query_len)
+    return torch_ref.gated_unit_step(u, ra, ra_bias, ri, ri_bias, rate, gate, gate_bias, state, slots, query_start_loc,
+                                     seq_lens)

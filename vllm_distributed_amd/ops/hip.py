@@ -69,13 +69,19 @@ def load() -> ctypes.CDLL:
         "vdamd_scalar_norm_residual": [P, P, P, P, P, F, I, I, L, I, I, P],
         "vdamd_poly_norm": [P, P, P, F, I, I, L, I, P],
         "vdamd_conv_norm_cache": [P, L] + [P] * 16 + [I] * 8 + [F, I, P, I, I, P],
-        "vdamd_short_conv_act": [P, L, P, L, P, P, P, P, P, P, P] + [I] * 6 + [P, I, I, P],
+        "vdamd_short_conv_act": [P, L, P, L, P, P, P, P, P, P, P] + [I] * 6 + [P, I, P, I, P],
+        "vdamd_rotate_norm_cache": [P, P, L, P, I, F, I, F] + [P] * 6 + [I] * 7 + [P],
         "vdamd_window_bias_attention": [P, P, P, P, L, P, P, P, P, P, P, P, P, L, P] + [I] * 10 + [F, F, I, I, I, I, P],
         "vdamd_selective_scan": [P, P, L, P, L, P, P, P, P, P, P, P] + [I] * 7 + [P],
         "vdamd_act_gate_group_norm": [P, P, P, L, P, F, I, I, I, I, P],
         "vdamd_joint_norm_cache": [P, P, L, P, P, F, P, F, I, P, P, P] + [I] * 6 + [P],
         "vdamd_mix_heads": [P, P, P, I, I, I, I, I, P],
-        "vdamd_residual_rms": [P, L, P, L, P, L, P, L, P, L, P, P, F, F, I, I, I, I, I, I, P],
+        "vdamd_residual_rms": [P, L, P, L, P, L, P, L, P, L, P, P, F, F, I, I, I, I, I, I, F, P],
+        "vdamd_gelu_and_mul": [P, P, L, I, I, I, I, P],
+        "vdamd_channel_scan": [P, P, L, P, L, P, L, P, L] + [P] * 7 + [I] * 6 + [P],
+        "vdamd_block_gates_mfma_ok": [I, I],
+        "vdamd_block_gates": [P] * 10 + [L, P, P, P, P, I, I, I, I, P],
+        "vdamd_gated_unit_scan": [P, P, P, P, L, P, P, P, P, P, I, I, I, I, P],
         "vdamd_gelu_mul_rows": [P, P, L, P, L, P, I, I, I, I, I, P],
         "vdamd_sigmoid_mul": [P, L, P, L, P, L, F, I, I, I, P],
         "vdamd_gelu": [P, P, L, I, I, P],
@@ -83,7 +89,7 @@ def load() -> ctypes.CDLL:
         "vdamd_gated_delta_rule": [P, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "vdamd_embed_scaled": [P, P, P, F, I, I, I, I, P],
         "vdamd_layer_norm_to": [P, P, L, P, L, P, P, F, I, I, I, I, I, P],
-        "vdamd_gated_rms_norm": [P, L, P, P, P, L, F, I, I, I, F, I, I, P],
+        "vdamd_gated_rms_norm": [P, L, P, P, P, L, F, I, I, I, F, I, I, I, P],
         "vdamd_clamped_glu": [P, P, L, I, I, F, F, I, P],
         "vdamd_relu_squared": [P, P, L, I, P],
         "vdamd_expert_epilogue": [P, P, P, L, P, P, I, I, P, P, L, I, I, I, P],
@@ -1454,7 +1460,8 @@ def decay_linear_attention(x: torch.Tensor, num_heads: int, dim: int, vdim: int,
 
 
 def gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, eps: float,
-                   out_dtype: torch.dtype, group: int = 0, scale: float = 1.0, out=None) -> torch.Tensor:
+                   out_dtype: torch.dtype, group: int = 0, scale: float = 1.0, out=None,
+                   silu: bool = False) -> torch.Tensor:
     t, n = o.shape
     assert o.dtype == torch.float32 and o.is_contiguous() and gate.shape == (t, n) and gate.stride(1) == 1
     group = int(group or 0)
@@ -1464,7 +1471,8 @@ def gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, ep
     assert out.dim() == 2 and out.shape == (t, n) and out.stride(1) == 1
     _check(_LIB.vdamd_gated_rms_norm(out.data_ptr(), out.stride(0), o.data_ptr(),
                                      _f32_vec(weight, group or n, "weight").data_ptr(), gate.data_ptr(), gate.stride(0),
-                                     float(eps), t, n, group, float(scale), _dt(gate), _dt(out), _stream()),
+                                     float(eps), t, n, group, float(scale), 1 if silu else 0, _dt(gate), _dt(out),
+                                     _stream()),
            "gated_rms_norm")
     return out
 
@@ -1574,7 +1582,7 @@ def _rows2d(t: torch.Tensor, name: str) -> torch.Tensor:
     return t
 
 
-def _residual_rms(x, a, b, y, post_w, w, eps, out_dtype, offset, normed) -> torch.Tensor:
+def _residual_rms(x, a, b, y, post_w, w, eps, out_dtype, offset, normed, post_scale: float = 1.0) -> torch.Tensor:
     rows, h = _rows2d(x, "x").shape
     adds = a is not None or y is not None
     if adds:
@@ -1592,7 +1600,8 @@ def _residual_rms(x, a, b, y, post_w, w, eps, out_dtype, offset, normed) -> torc
         out.data_ptr(), h, x.data_ptr(), x.stride(0), _ptr(a), 0 if a is None else a.stride(0), _ptr(b),
         0 if b is None else b.stride(0), _ptr(y), 0 if y is None else y.stride(0),
         _ptr(_f32_vec(post_w, h, "post_weight")) if y is not None else None, _ptr(_f32_vec(w, h, "weight")),
-        float(offset), float(eps), rows, h, 1 if normed else 0, _dt(x), in_dt, _DT[out_dtype], _stream()), "residual_rms")
+        float(offset), float(eps), rows, h, 1 if normed else 0, _dt(x), in_dt, _DT[out_dtype],
+        float(post_scale), _stream()), "residual_rms")
     return out
 
 
@@ -1609,9 +1618,10 @@ def add_rms_norm_to(residual, a, b, weight, eps: float, out_dtype, offset: float
 
 
 def norm_add_norm(y, post_weight, residual, next_weight, eps: float, out_dtype, next_offset: float = 0.0,
-                  next_normed: bool = True):
+                  next_normed: bool = True, post_scale: float = 1.0):
     assert residual.is_contiguous()
-    return _residual_rms(residual, None, None, y, post_weight, next_weight, eps, out_dtype, next_offset, next_normed)
+    return _residual_rms(residual, None, None, y, post_weight, next_weight, eps, out_dtype, next_offset, next_normed,
+                         post_scale)
 
 
 def gelu_mul_rows(g: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, col: int) -> torch.Tensor:
@@ -1643,7 +1653,8 @@ def gelu(x: torch.Tensor, tanh: bool) -> torch.Tensor:
 
 
 def short_conv_act(x, channels: int, conv_weight, state, slots, query_start_loc, seq_lens, token_seq, positions,
-                   silu: bool, has_prefill: bool = True, bias=None, residual: bool = False) -> torch.Tensor:
+                   silu: bool, has_prefill: bool = True, bias=None, residual: bool = False,
+                   in_bias=None) -> torch.Tensor:
     t = _rows2d(x, "x").shape[0]
     c, taps = int(channels), conv_weight.shape[0]
     r = max(taps - 1, 1)
@@ -1662,35 +1673,39 @@ def short_conv_act(x, channels: int, conv_weight, state, slots, query_start_loc,
         _i32(slots, "slots").data_ptr(), _i32(query_start_loc, "query_start_loc").data_ptr(),
         _i32(seq_lens, "seq_lens").data_ptr(), _ptr(_i32(token_seq, "token_seq")),
         _i32(positions, "positions").data_ptr(), t, b, c, taps, 1 if silu else 0, 1 if has_prefill else 0,
-        _ptr(_f32_vec(bias, c, "bias")), 1 if residual else 0, _dt(x), _stream()), "short_conv_act")
+        _ptr(_f32_vec(bias, c, "bias")), 1 if residual else 0, _ptr(_f32_vec(in_bias, c, "in_bias")), _dt(x), _stream()),
+        "short_conv_act")
     return out
 
 
 def gated_delta_rule(x, num_heads: int, num_qk_heads: int, dim: int, vdim: int, beta, dt, dt_bias, a_log, state, slots,
                      query_start_loc, seq_lens, norm_eps: float = 1e-6, max_query_len: int = 0,
                      parts: int = 0) -> torch.Tensor:
-    """``max_query_len`` (0: unknown) only helps the kernel choose its tiling; ``parts`` forces one (benchmarks)."""
+    """``max_query_len`` (0: unknown) only helps the kernel choose its tiling; ``parts`` forces one (benchmarks).
+    ``dt[T, H]``: one decay per head."""
     t = _rows2d(x, "x").shape[0]
     h, g = int(num_heads), int(num_qk_heads)
     b = seq_lens.shape[0]
     assert h % g == 0 and 0 < dim <= 256 and x.shape[1] >= 2 * g * dim + h * vdim
     assert _rows2d(beta, "beta").shape[0] >= t and beta.shape[1] == h and beta.dtype == x.dtype
-    assert _rows2d(dt, "dt").shape[0] >= t and dt.shape[1] == h * dim and dt.dtype == x.dtype
+    per_head = dt.shape[1] == h
+    assert _rows2d(dt, "dt").shape[0] >= t and (per_head or dt.shape[1] == h * dim) and dt.dtype == x.dtype
     assert state is not None and state.dtype == torch.float32 and state.is_contiguous()
     assert tuple(state.shape[1:]) == (h, dim, vdim), (tuple(state.shape), (h, dim, vdim))
     assert slots.shape[0] == b and query_start_loc.shape[0] >= b + 1
     dev = x.device
     qn = torch.empty((t, g, dim), dtype=torch.float32, device=dev)
     kn = torch.empty((t, g, dim), dtype=torch.float32, device=dev)
-    decay = torch.empty((t, h, dim), dtype=torch.float32, device=dev)
-    bsig = torch.empty((t, 2, h), dtype=torch.float32, device=dev)   # sigmoid(beta) | k.q of the head's group
+    decay = None if per_head else torch.empty((t, h, dim), dtype=torch.float32, device=dev)
+    # sigmoid(beta) | k.q of the head's group (| the head's decay)
+    bsig = torch.empty((t, 3 if per_head else 2, h), dtype=torch.float32, device=dev)
     out = torch.empty((t, h * vdim), dtype=torch.float32, device=dev)
     _check(_LIB.vdamd_delta_rule_prep(
-        qn.data_ptr(), kn.data_ptr(), decay.data_ptr(), bsig.data_ptr(), x.data_ptr(), x.stride(0), beta.data_ptr(),
-        beta.stride(0), dt.data_ptr(), dt.stride(0), _f32_vec(dt_bias, h * dim, "dt_bias").data_ptr(),
+        qn.data_ptr(), kn.data_ptr(), _ptr(decay), bsig.data_ptr(), x.data_ptr(), x.stride(0), beta.data_ptr(),
+        beta.stride(0), dt.data_ptr(), dt.stride(0), _f32_vec(dt_bias, dt.shape[1], "dt_bias").data_ptr(),
         _f32_vec(a_log, h, "a_log").data_ptr(), t, h, g, dim, float(norm_eps), _dt(x), _stream()), "delta_rule_prep")
     _check(_LIB.vdamd_gated_delta_rule(
-        out.data_ptr(), x.data_ptr(), x.stride(0), 2 * g * dim, qn.data_ptr(), kn.data_ptr(), decay.data_ptr(),
+        out.data_ptr(), x.data_ptr(), x.stride(0), 2 * g * dim, qn.data_ptr(), kn.data_ptr(), _ptr(decay),
         bsig.data_ptr(), state.data_ptr(), _i32(slots, "slots").data_ptr(),
         _i32(query_start_loc, "query_start_loc").data_ptr(), _i32(seq_lens, "seq_lens").data_ptr(), b, h, g, dim, vdim,
         int(max_query_len), int(parts), _dt(x), _stream()), "gated_delta_rule")
@@ -1762,3 +1777,118 @@ def mix_heads(o: torch.Tensor, talk: torch.Tensor, out_dtype: torch.dtype) -> to
     _check(_LIB.vdamd_mix_heads(out.data_ptr(), o.data_ptr(), _f32_vec(talk, h * h, "talk").data_ptr(), t, h, g, dv,
                                 _dt(out), _stream()), "mix_heads")
     return out
+
+
+# ------------------------------------------------ rotation in front of a head norm, a selective scan per channel, a
+# ------------------------------------------------ gated linear unit recurrence
+def rotate_norm_cache(x, num_heads: int, num_kv_heads: int, dim: int, vdim: int, inv_freq, rot_scale: float,
+                      interleaved: bool, eps: float, q_norm, k_norm, positions, k_cache, v_cache,
+                      slot_mapping) -> torch.Tensor:
+    t = _rows2d(x, "x").shape[0]
+    h, g, d, dv = int(num_heads), int(num_kv_heads), int(dim), int(vdim)
+    assert x.shape[1] >= (h + g) * d + g * dv and positions.shape[0] >= t and h % g == 0 and d <= UNIT_MAX_WIDTH
+    half = 0 if inv_freq is None else int(inv_freq.numel())
+    assert 2 * half <= d
+    bs = 0
+    if k_cache is not None:
+        bs = k_cache.shape[2]
+        assert k_cache.dtype == v_cache.dtype == x.dtype and k_cache.is_contiguous() and v_cache.is_contiguous()
+        assert tuple(k_cache.shape[1:]) == (g, bs, d) and bs % 8 == 0
+        assert tuple(v_cache.shape) == (k_cache.shape[0], g, bs // 8, dv, 8)
+        assert slot_mapping.shape[0] >= t
+    q = torch.empty((t, h, d), dtype=x.dtype, device=x.device)
+    _check(_LIB.vdamd_rotate_norm_cache(
+        q.data_ptr(), x.data_ptr(), x.stride(0), _ptr(_f32_vec(inv_freq, half, "inv_freq")) if half else None, half,
+        float(rot_scale), 1 if interleaved else 0, float(eps), _ptr(_f32_vec(q_norm, d, "q_norm")),
+        _ptr(_f32_vec(k_norm, d, "k_norm")), _i32(positions, "positions").data_ptr(), _ptr(k_cache), _ptr(v_cache),
+        _ptr(_i32(slot_mapping, "slot_mapping") if k_cache is not None else None), t, h, g, d, dv, int(bs), _dt(x),
+        _stream()), "rotate_norm_cache")
+    return q
+
+
+def gelu_and_mul(x: torch.Tensor, tanh: bool = True) -> torch.Tensor:
+    f = x.shape[-1] // 2
+    x2 = x.reshape(-1, 2 * f)
+    if x2.stride(1) != 1:
+        x2 = x2.contiguous()
+    out = torch.empty((x2.shape[0], f), dtype=x.dtype, device=x.device)
+    _check(_LIB.vdamd_gelu_and_mul(out.data_ptr(), x2.data_ptr(), x2.stride(0), x2.shape[0], f, 1 if tanh else 0, _dt(x2),
+                                   _stream()), "gelu_and_mul")
+    return out.view(x.shape[:-1] + (f,))
+
+
+def channel_scan(u, dt, bc, n_state: int, a_log, dt_bias, d_skip, gate, state, slots, query_start_loc, seq_lens,
+                 max_query_len: int = 0) -> torch.Tensor:
+    """``max_query_len`` (0: unknown) only helps the kernel choose its launch; 1 must be true."""
+    t, c = _rows2d(u, "u").shape
+    n, b = int(n_state), seq_lens.shape[0]
+    if not 0 < n <= 256:
+        raise NotImplementedError(f"a selective scan with {n} states per channel (at most 256)")
+    assert _rows2d(dt, "dt").shape[0] >= t and dt.shape[1] == c and dt.dtype in (u.dtype, torch.float32)
+    assert _rows2d(bc, "bc").shape[0] >= t and bc.shape[1] >= 2 * n and bc.dtype == u.dtype
+    if gate is not None:
+        assert _rows2d(gate, "gate").shape[0] >= t and gate.shape[1] == c and gate.dtype == u.dtype
+    assert state is not None and state.dtype == torch.float32 and state.is_contiguous()
+    assert tuple(state.shape[1:]) == (c, n), (tuple(state.shape), (c, n))
+    assert slots.shape[0] == b and query_start_loc.shape[0] >= b + 1
+    assert max_query_len != 1 or t <= b
+    out = torch.empty((t, c), dtype=u.dtype, device=u.device)
+    _check(_LIB.vdamd_channel_scan(
+        out.data_ptr(), u.data_ptr(), u.stride(0), dt.data_ptr(), dt.stride(0), bc.data_ptr(), bc.stride(0), _ptr(gate),
+        0 if gate is None else gate.stride(0), _f32_vec(a_log, c * n, "a_log").data_ptr(),
+        _ptr(_f32_vec(dt_bias, c, "dt_bias")), _ptr(_f32_vec(d_skip, c, "d_skip")), state.data_ptr(),
+        _i32(slots, "slots").data_ptr(), _i32(query_start_loc, "query_start_loc").data_ptr(),
+        _i32(seq_lens, "seq_lens").data_ptr(), b, c, n, int(max_query_len), _dt(u), _dt(dt), _stream()), "channel_scan")
+    return out
+
+
+def _block_gates(u, ra, ra_bias, ri, ri_bias, rate, a, drive, out, gate, gate_bias, state, slots, seq_lens) -> None:
+    t, w = _rows2d(u, "u").shape
+    n = ra.shape[1]
+    assert u.is_contiguous() and ra.is_contiguous() and ri.is_contiguous() and ra.dtype == ri.dtype == u.dtype
+    assert ra.shape == ri.shape == (w // n, n, n) and w % n == 0
+    _check(_LIB.vdamd_block_gates(
+        _ptr(a), _ptr(drive), u.data_ptr(), ra.data_ptr(), _f32_vec(ra_bias, w, "ra_bias").data_ptr(), ri.data_ptr(),
+        _f32_vec(ri_bias, w, "ri_bias").data_ptr(), _f32_vec(rate, w, "rate").data_ptr(), _ptr(out), _ptr(gate),
+        0 if gate is None else gate.stride(0), _ptr(_f32_vec(gate_bias, w, "gate_bias")), _ptr(state), _ptr(slots),
+        _ptr(seq_lens), t, w, n, _dt(u), _stream()), "block_gates")
+
+
+def block_gates(u, ra, ra_bias, ri, ri_bias, rate):
+    a = torch.empty(u.shape, dtype=torch.float32, device=u.device)
+    drive = torch.empty_like(a)
+    _block_gates(u, ra, ra_bias, ri, ri_bias, rate, a, drive, None, None, None, None, None, None)
+    return a, drive
+
+
+def gated_unit_scan(a, drive, gate, gate_bias, state, slots, query_start_loc, seq_lens,
+                    max_query_len: int = 0) -> torch.Tensor:
+    t, w = a.shape
+    b = seq_lens.shape[0]
+    assert a.dtype == drive.dtype == torch.float32 and a.is_contiguous() and drive.is_contiguous() and drive.shape == a.shape
+    assert _rows2d(gate, "gate").shape[0] >= t and gate.shape[1] == w
+    assert state is not None and state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (w,)
+    assert slots.shape[0] == b and query_start_loc.shape[0] >= b + 1
+    out = torch.empty((t, w), dtype=gate.dtype, device=a.device)
+    _check(_LIB.vdamd_gated_unit_scan(
+        out.data_ptr(), a.data_ptr(), drive.data_ptr(), gate.data_ptr(), gate.stride(0),
+        _ptr(_f32_vec(gate_bias, w, "gate_bias")), state.data_ptr(), _i32(slots, "slots").data_ptr(),
+        _i32(query_start_loc, "query_start_loc").data_ptr(), _i32(seq_lens, "seq_lens").data_ptr(), b, w,
+        int(max_query_len), _dt(gate), _stream()), "gated_unit_scan")
+    return out
+
+
+def gated_unit_step(u, ra, ra_bias, ri, ri_bias, rate, gate, gate_bias, state, slots, query_start_loc, seq_lens,
+                    max_query_len: int = 0) -> torch.Tensor:
+    t, w = u.shape
+    if (max_query_len == 1 and t == seq_lens.shape[0] and gate.stride(0) % 4 == 0 and gate.data_ptr() % 8 == 0
+            and _LIB.vdamd_block_gates_mfma_ok(int(ra.shape[1]), _dt(u))):
+        # every row is its sequence's only one: gates, state and output gate in one launch
+        assert state is not None and state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (w,)
+        assert _rows2d(gate, "gate").shape == (t, w) and gate.dtype == u.dtype and slots.shape[0] == t
+        out = torch.empty((t, w), dtype=u.dtype, device=u.device)
+        _block_gates(u, ra, ra_bias, ri, ri_bias, rate, None, None, out, gate, gate_bias, state, _i32(slots, "slots"),
+                     _i32(seq_lens, "seq_lens"))
+        return out
+    a, drive = block_gates(u, ra, ra_bias, ri, ri_bias, rate)
+    return gated_unit_scan(a, drive, gate, gate_bias, state, slots, query_start_loc, seq_lens, max_query_len)

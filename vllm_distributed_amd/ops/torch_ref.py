@@ -467,12 +467,15 @@ def poly_norm(z: torch.Tensor, coef: torch.Tensor, eps: float) -> torch.Tensor:
 
 
 def short_conv(x: torch.Tensor, weight: torch.Tensor, state: torch.Tensor, slots: torch.Tensor,
-               query_start_loc: torch.Tensor, seq_lens: torch.Tensor) -> torch.Tensor:
+               query_start_loc: torch.Tensor, seq_lens: torch.Tensor,
+               in_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal per-channel convolution over time of the packed rows ``x[T, C]`` with tap-major ``weight[taps, C]``:
     ``y_t = sum_j weight[j] * u_(t - taps + 1 + j)``, zero before a sequence's first position.  Sequence ``i``
     owns rows ``query_start_loc[i]:query_start_loc[i+1]``, the last positions of its ``seq_lens[i]`` tokens; the
     ``taps - 1`` inputs in front of them come from ``state[slots[i]]`` (``[slots, taps - 1, C]``, oldest first),
-    which is left holding the last ``taps - 1`` inputs of the sequence.  Returns fp32 ``[T, C]``."""
+    which is left holding the last ``taps - 1`` inputs of the sequence.  ``in_bias[C]`` is added to every input that
+    exists (positions before the sequence's start stay zero; the state holds inputs without it).  Returns fp32
+    ``[T, C]``."""
     taps = weight.shape[0]
     r = taps - 1
     y = torch.empty(x.shape, dtype=torch.float32, device=x.device)
@@ -492,6 +495,9 @@ def short_conv(x: torch.Tensor, weight: torch.Tensor, state: torch.Tensor, slots
         acc = torch.zeros((n, x.shape[1]), dtype=torch.float32, device=x.device)
         for j in range(taps):
             acc += wf[j] * u[j:j + n]
+            if in_bias is not None:
+                absent = min(max(r - start - j, 0), n)          # rows whose tap j reaches in front of the sequence
+                acc[absent:] += wf[j] * in_bias.float()
         y[s:e] = acc
         if r:
             state[sl[i]] = u[u.shape[0] - r:].to(state.dtype)
@@ -654,8 +660,9 @@ def decay_linear_attention(x: torch.Tensor, num_heads: int, dim: int, vdim: int,
 
 def gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, eps: float,
                    out_dtype: torch.dtype, group: int = 0, scale: float = 1.0,
-                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``o / sqrt(mean(o^2) + eps) * weight * sigmoid(gate) * scale`` in fp32 arithmetic, the mean over whole rows or,
+                   out: Optional[torch.Tensor] = None, silu: bool = False) -> torch.Tensor:
+    """``o / sqrt(mean(o^2) + eps) * weight * sigmoid(gate) * scale`` (``silu``: times ``silu(gate)`` instead of
+    ``sigmoid(gate)``) in fp32 arithmetic, the mean over whole rows or,
     with ``group > 0``, over each run of ``group`` values (``weight[group]`` then serves every run).  ``out``: a
     ``[T, N]`` view (rows may be strided) that receives the result."""
     of = o.float()
@@ -664,7 +671,7 @@ def gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, ep
         y = (g * torch.rsqrt(g.pow(2).mean(-1, keepdim=True) + eps) * weight.float()).flatten(-2)
     else:
         y = of * torch.rsqrt(of.pow(2).mean(-1, keepdim=True) + eps) * weight.float()
-    y = y * torch.sigmoid(gate.float()) * scale
+    y = y * (F.silu(gate.float()) if silu else torch.sigmoid(gate.float())) * scale
     if out is not None:
         out.copy_(y)
         return out
@@ -814,10 +821,10 @@ def add_rms_norm_to(residual: torch.Tensor, a: Optional[torch.Tensor], b: Option
 
 def norm_add_norm(y: torch.Tensor, post_weight: torch.Tensor, residual: torch.Tensor,
                   next_weight: Optional[torch.Tensor], eps: float, out_dtype: torch.dtype, next_offset: float = 0.0,
-                  next_normed: bool = True) -> Optional[torch.Tensor]:
-    """``residual += rms_norm(y) * post_weight`` in place on the fp32 residual stream; then what
+                  next_normed: bool = True, post_scale: float = 1.0) -> Optional[torch.Tensor]:
+    """``residual += post_scale * rms_norm(y) * post_weight`` in place on the fp32 residual stream; then what
     ``add_rms_norm_to(residual, None, None, next_weight, ...)`` returns."""
-    residual.add_(rms_norm_to(y, post_weight, eps, torch.float32))
+    residual.add_(rms_norm_to(y, post_weight, eps, torch.float32), alpha=post_scale)
     if not next_normed:
         return residual.to(out_dtype)
     return rms_norm_to(residual, next_weight, eps, out_dtype, next_offset)
@@ -844,11 +851,13 @@ def sigmoid_mul(o: torch.Tensor, gate: torch.Tensor, scale: float = 1.0, out: Op
 
 def short_conv_act(x: torch.Tensor, channels: int, conv_weight: torch.Tensor, state: torch.Tensor, slots: torch.Tensor,
                    query_start_loc: torch.Tensor, seq_lens: torch.Tensor, silu: bool,
-                   bias: Optional[torch.Tensor] = None, residual: bool = False) -> torch.Tensor:
-    """``short_conv`` over the first ``channels`` columns of ``x`` (the state moves on), plus ``bias[channels]``,
+                   bias: Optional[torch.Tensor] = None, residual: bool = False,
+                   in_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``short_conv`` over the first ``channels`` columns of ``x`` (``in_bias`` added to every input that exists; the
+    state moves on), plus ``bias[channels]``,
     through SiLU when ``silu``; with ``residual`` the input itself is added at the end (``x + conv(x)``);
     ``[T, channels]`` in ``x``'s dtype."""
-    y = short_conv(x[:, :channels], conv_weight, state, slots, query_start_loc, seq_lens)
+    y = short_conv(x[:, :channels], conv_weight, state, slots, query_start_loc, seq_lens, in_bias)
     if bias is not None:
         y = y + bias.float()
     if silu:
@@ -865,7 +874,8 @@ def gated_delta_rule(x: torch.Tensor, num_heads: int, num_qk_heads: int, dim: in
     """The gated delta rule over the packed rows ``x[T, C]`` = ``[q (Hqk * dim) | k (Hqk * dim) | v (H * vdim)]``;
     value head ``h`` reads q / k head ``h // (H / Hqk)``.  Per row: q and k become unit vectors
     (``u / sqrt(sum(u^2) + norm_eps)``), q times ``dim^-0.5``; ``b = sigmoid(beta[t, h])``; one decay per head and
-    key channel ``g = exp(-exp(a_log[h]) * softplus(dt[t, h, :] + dt_bias[h, :]))``; then ``S <- g * S`` by rows,
+    key channel ``g = exp(-exp(a_log[h]) * softplus(dt[t, h, :] + dt_bias[h, :]))``, or with ``dt[T, H]`` and
+    ``dt_bias[H]`` one per head; then ``S <- g * S`` by rows,
     ``u = b (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q``.  ``S`` is ``state[slots[i]]`` (``[slots, H, dim, vdim]``
     fp32) for sequence ``i``, taken as zero when the rows start at position 0 whatever the slot held, and left holding
     the state after the sequence's last row.  fp32 arithmetic; returns fp32 ``[T, H * vdim]``."""
@@ -880,7 +890,7 @@ def gated_delta_rule(x: torch.Tensor, num_heads: int, num_qk_heads: int, dim: in
     v = xf[:, 2 * qs:].reshape(t, h, vdim)
     b = torch.sigmoid(beta[:t].float())
     decay = torch.exp(-torch.exp(a_log.float()).view(1, h, 1)
-                      * F.softplus(dt[:t].float().reshape(t, h, dim) + dt_bias.float().view(1, h, dim)))
+                      * F.softplus(dt[:t].float().reshape(t, h, -1) + dt_bias.float().view(1, h, -1), threshold=30.0))
     out = torch.zeros((t, h, vdim), dtype=torch.float32, device=x.device)
     qsl, sls, sl = query_start_loc.tolist(), seq_lens.tolist(), slots.tolist()
     for i, n_ctx in enumerate(sls):
@@ -1010,3 +1020,124 @@ def mix_heads(o: torch.Tensor, talk: torch.Tensor, out_dtype: torch.dtype) -> to
     own = torch.arange(h, device=o.device) // (h // c)
     picked = o.float()[:, :, own, :]                                # [T, g, h, Dv]
     return torch.einsum("hg,tghd->thd", talk.float(), picked).reshape(t, h * dv).to(out_dtype)
+
+
+# ------------------------------------------------ rotation in front of a head norm, a selective scan per channel, a
+# ------------------------------------------------ gated linear unit recurrence
+def rotate_norm_cache(x: torch.Tensor, num_heads: int, num_kv_heads: int, dim: int, vdim: int,
+                      inv_freq: Optional[torch.Tensor], rot_scale: float, interleaved: bool, eps: float,
+                      q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], positions: torch.Tensor,
+                      k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor],
+                      slot_mapping: Optional[torch.Tensor]) -> torch.Tensor:
+    """What lies between the fused projection ``x[T, >= C]`` = ``[q (H * dim) | k (Hkv * dim) | v (Hkv * vdim)]`` and the
+    attention of a layer that rotates its heads BEFORE it norms them: the first ``2 * len(inv_freq)`` values of every
+    q and k head turned by ``positions[t] * inv_freq[i]`` (cos and sin times ``rot_scale``; ``interleaved`` pairs
+    neighbours), then the RMS norm of each head (``eps``; ``q_norm`` / ``k_norm`` ``[dim]`` gains or None: none), k and
+    v into ``k_cache[blocks, Hkv, block, dim]`` and ``v_cache[blocks, Hkv, block / 8, vdim, 8]``.  fp32 arithmetic;
+    returns ``q[T, H, dim]`` in ``x``'s dtype."""
+    t = x.shape[0]
+    qs, ks = num_heads * dim, num_kv_heads * dim
+    q = x[:, :qs].float().reshape(t, num_heads, dim)
+    k = x[:, qs:qs + ks].float().reshape(t, num_kv_heads, dim)
+    if inv_freq is not None and inv_freq.numel():
+        q = rotate_pairs_first(q, positions[:t], inv_freq, rot_scale, interleaved)
+        k = rotate_pairs_first(k, positions[:t], inv_freq, rot_scale, interleaved)
+    q, k = rms_norm_to(q, q_norm, eps, torch.float32), rms_norm_to(k, k_norm, eps, torch.float32)
+    if k_cache is not None:
+        v = x[:, qs + ks:qs + ks + num_kv_heads * vdim].reshape(t, num_kv_heads, vdim)
+        bs = k_cache.shape[2]
+        valid = slot_mapping[:t] >= 0
+        sm = slot_mapping[:t][valid].long()
+        blk, off = sm // bs, sm % bs
+        k_cache[blk, :, off, :] = k[valid].to(k_cache.dtype)
+        v_cache[blk, :, off // V_GROUP, :, off % V_GROUP] = v[valid].to(v_cache.dtype)
+    return q.to(x.dtype)
+
+
+def gelu_and_mul(x: torch.Tensor, tanh: bool = True) -> torch.Tensor:
+    """``gelu(x[..., :F]) * x[..., F:]`` in fp32 arithmetic, result in ``x``'s dtype."""
+    f = x.shape[-1] // 2
+    return (F.gelu(x[..., :f].float(), approximate="tanh" if tanh else "none") * x[..., f:].float()).to(x.dtype)
+
+
+def channel_scan(u: torch.Tensor, dt: torch.Tensor, bc: torch.Tensor, n_state: int, a_log: torch.Tensor,
+                 dt_bias: Optional[torch.Tensor], d_skip: Optional[torch.Tensor], gate: Optional[torch.Tensor],
+                 state: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor,
+                 seq_lens: torch.Tensor) -> torch.Tensor:
+    """A selective scan in which every channel has a state vector and decays of its own: ``u[T, C]``, raw step sizes
+    ``dt[T, C]``, ``bc[T, >= 2N]`` = ``[B (N) | C (N)]`` shared by the channels, ``a_log[C, N]``.  Per row
+    ``d = softplus(dt[t, c] + dt_bias[c])``, ``S[c, n] <- exp(-exp(a_log[c, n]) d) S[c, n] + d u[c] B[n]``,
+    ``y[c] = sum_n S[c, n] C[n] + d_skip[c] u[c]``, times ``silu(gate[t, c])`` when a gate is given.  ``S`` is
+    ``state[slots[i]]`` (``[slots, C, N]`` fp32) for sequence ``i``, taken as zero when the rows start at position 0
+    whatever the slot held, and left holding the state after the sequence's last row.  fp32 arithmetic; returns
+    ``[T, C]`` in ``u``'s dtype."""
+    t, n = u.shape[0], n_state
+    uf = u.float()
+    d = dt[:t].float()
+    d = F.softplus(d if dt_bias is None else d + dt_bias.float(), threshold=30.0)
+    bm, cm = bc[:t, :n].float(), bc[:t, n:2 * n].float()
+    rate = torch.exp(a_log.float())
+    y = torch.zeros_like(uf)
+    qsl, sls, sl = query_start_loc.tolist(), seq_lens.tolist(), slots.tolist()
+    for i, n_ctx in enumerate(sls):
+        s, e = qsl[i], qsl[i + 1]
+        if e == s:
+            continue
+        st = state[sl[i]].float().clone() if n_ctx - (e - s) > 0 else torch.zeros_like(state[sl[i]], dtype=torch.float32)
+        for r in range(s, e):
+            st = torch.exp(-rate * d[r].unsqueeze(1)) * st + (d[r] * uf[r]).unsqueeze(1) * bm[r]
+            y[r] = st @ cm[r]
+        state[sl[i]] = st.to(state.dtype)
+    if d_skip is not None:
+        y = y + d_skip.float() * uf
+    if gate is not None:
+        y = y * F.silu(gate[:t].float())
+    return y.to(u.dtype)
+
+
+def block_gates(u: torch.Tensor, ra: torch.Tensor, ra_bias: torch.Tensor, ri: torch.Tensor, ri_bias: torch.Tensor,
+                rate: torch.Tensor):
+    """The gates of a gated linear unit recurrence over ``u[T, W]`` in ``blocks`` equal runs of channels, each run with
+    square matrices ``ra[b]`` and ``ri[b]`` (``[blocks, n, n]``, out by in) and biases ``[W]``: ``r = sigmoid(ra u +
+    bias)``, ``i = sigmoid(ri u + bias)``; ``log_a = -rate * r``.  Returns fp32 ``a = exp(log_a)`` and
+    ``sqrt(1 - a^2) * i * u``, both ``[T, W]``."""
+    t, width = u.shape
+    nb, n = ra.shape[0], ra.shape[1]
+    uf = u.float()
+    ub = uf.reshape(t, nb, n).transpose(0, 1)
+
+    def gate(w, b):
+        z = torch.bmm(ub, w.float().transpose(1, 2).contiguous()).transpose(0, 1).reshape(t, width)
+        return torch.sigmoid(z + b.float())
+    log_a = -rate.float() * gate(ra, ra_bias)
+    return torch.exp(log_a), torch.sqrt(-torch.expm1(2.0 * log_a)) * gate(ri, ri_bias) * uf
+
+
+def gated_unit_scan(a: torch.Tensor, drive: torch.Tensor, gate: torch.Tensor, gate_bias: Optional[torch.Tensor],
+                    state: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor,
+                    seq_lens: torch.Tensor) -> torch.Tensor:
+    """``S_t = a_t S_(t-1) + drive_t`` per channel (``a``, ``drive`` fp32 ``[T, W]``), times
+    ``gelu_tanh(gate[t] + gate_bias)``; ``S`` is ``state[slots[i]]`` (``[slots, W]`` fp32) for sequence ``i``, taken as zero
+    when the rows start at position 0 whatever the slot held, and left holding the state after the sequence's last row.
+    fp32 arithmetic; returns ``[T, W]`` in ``gate``'s dtype."""
+    y = torch.zeros_like(drive)
+    qsl, sls, sl = query_start_loc.tolist(), seq_lens.tolist(), slots.tolist()
+    for i, n_ctx in enumerate(sls):
+        s, e = qsl[i], qsl[i + 1]
+        if e == s:
+            continue
+        st = state[sl[i]].float().clone() if n_ctx - (e - s) > 0 else torch.zeros_like(state[sl[i]], dtype=torch.float32)
+        for r in range(s, e):
+            st = a[r] * st + drive[r]
+            y[r] = st
+        state[sl[i]] = st.to(state.dtype)
+    z = gate[:y.shape[0]].float()
+    return (y * gelu_tanh_f(z if gate_bias is None else z + gate_bias.float())).to(gate.dtype)
+
+
+def gated_unit_step(u: torch.Tensor, ra: torch.Tensor, ra_bias: torch.Tensor, ri: torch.Tensor, ri_bias: torch.Tensor,
+                    rate: torch.Tensor, gate: torch.Tensor, gate_bias: Optional[torch.Tensor], state: torch.Tensor,
+                    slots: torch.Tensor, query_start_loc: torch.Tensor, seq_lens: torch.Tensor) -> torch.Tensor:
+    """``block_gates`` and ``gated_unit_scan`` one after the other."""
+    a, drive = block_gates(u, ra, ra_bias, ri, ri_bias, rate)
+    return gated_unit_scan(a, drive, gate, gate_bias, state, slots, query_start_loc, seq_lens)
