@@ -139,10 +139,10 @@ def _parse():
     ap.add_argument("--alt-parallelism", type=str, default="pp",
                     help="second layout measured in a child process after the headline when N > 1 ('none' = skip)")
     ap.add_argument("--alt-timeout", type=float, default=900.0)
-    ap.add_argument("--family-compare", type=str, default=None, choices=[None, "tavulix", "kabapel", "gosizen", "nalasun"],
+    ap.add_argument("--family-compare", type=str, default=None, choices=[None, "tavulix", "kabapel", "gosizen", "nalasun", "kefurax"],
                     help="instead of the headline: prefill and decode throughput of this model family at a few layer "
                          "sizes beside the closest existing family at equal size (Tavulix: Gemma-2; Kabapel: "
-                         "DeepSeek-V2; Gosizen: Kabapel; Nalasun: Gosizen), random weights, one GPU")
+                         "DeepSeek-V2; Gosizen: Kabapel; Nalasun: Gosizen; Kefurax: Nalasun), random weights, one GPU")
     ap.add_argument("--compare-sizes", type=str, default="small,medium",
                     help="with --family-compare: which of small / medium / large to run")
     ap.add_argument("--compare-only", type=str, default=None,
@@ -322,6 +322,31 @@ def _nalasun_models(z: dict) -> dict:
     return {"nalasun": ("nalasun-tiny", nal), "gosizen": _gosizen_models(z)["gosizen"]}
 
 
+def _kefurax_models(z: dict) -> dict:
+    """The same layer sizes as a Kefurax config (attention beside the gated delta rule, a gated linear unit recurrence, a
+    selective scan per channel and the parallel layer again, in turn; a dense feed-forward of the width the other
+    family's active experts add up to) and as a Nalasun config (attention, delta rule, state-space recurrence around an
+    fp32 residual stream: the closest family the framework has)."""
+    vocab = 32000
+    cols = z["heads"] * z["vdim"]
+    mlp = {"kind": "dense", "ff": z["top"] * z["ff"] + z["shared"]}
+    par = {"left": {"heads": z["heads"], "kv_heads": max(z["heads"] // 4, 1), "dim": z["nope"], "vdim": z["vdim"],
+                    "scale": z["nope"] ** 0.5 / 4.0,
+                    "rot": {"base": 10000.0, "dims": z["nope"],
+                            "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}},
+           "right": {"heads": z["heads"], "kv_heads": z["heads"], "dim": z["nope"], "vdim": z["vdim"], "conv": 4},
+           "left_scale": 0.5, "right_scale": 0.5}
+    mixers = [("parallel", par), ("rglru", {"width": cols, "blocks": z["heads"], "conv": 4}),
+              ("mamba1", {"inner": 2 * cols, "state": 16, "dt_rank": max(z["width"] // 16, 8), "conv": 4})]
+    order = [0, 1, 2, 0]
+    kef = {"architecture": "Kefurax", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-5},
+           "embedding": {"scale": z["width"] ** 0.5}, "residual_mult": 0.7,
+           "layers": [{"type": mixers[order[i % 4]][0], "mixer": mixers[order[i % 4]][1], "mlp": mlp}
+                      for i in range(z["layers"] if z["layers"] > 2 else 3)]}
+    nal = _nalasun_models(dict(z, layers=max(z["layers"], 3)))["nalasun"]
+    return {"kefurax": ("kefurax-tiny", kef), "nalasun": nal}
+
+
 def run_family_compare(args) -> None:
     """Prefill throughput (``prompts`` prompts of ``prompt`` tokens, one generated token each) and decode
     throughput (``batch`` sequences, 64 further tokens each; the prefill time measured the same way is taken off)
@@ -331,10 +356,11 @@ def run_family_compare(args) -> None:
     from vllm_distributed_amd import LLM, SamplingParams
     os.environ.setdefault("VLLM_LOGGING_LEVEL", "WARNING")
     rows = []
-    kabapel = args.family_compare in ("kabapel", "gosizen", "nalasun")
+    kabapel = args.family_compare in ("kabapel", "gosizen", "nalasun", "kefurax")
     for size in [s for s in args.compare_sizes.split(",") if s]:
         z = (KABAPEL_SIZES if kabapel else COMPARE_SIZES)[size]
-        by_family = {"gosizen": _gosizen_models, "nalasun": _nalasun_models, "kabapel": _kabapel_models}
+        by_family = {"gosizen": _gosizen_models, "nalasun": _nalasun_models, "kabapel": _kabapel_models,
+                     "kefurax": _kefurax_models}
         models = by_family[args.family_compare](z) if kabapel else _compare_models(z)
         for family, (base, over) in models.items():
             if args.compare_only and family != args.compare_only:

@@ -13,7 +13,9 @@
 //   gated_unit_scan   the same recurrence over prompt portions: 16 waves take 8 rows each of a 128-row chunk, scan them
 //                     locally, exchange (product of a, local end state) through LDS and apply the carried state - one
 //                     barrier per chunk, the next chunk's loads in flight
-// 1 - a^2 is formed as -expm1(2 log a): near a = 1 the plain difference would cancel.
+// 1 - a^2 is formed as -(e^(2 log a) - 1) without the cancellation a plain difference has near a = 1, and softplus keeps its
+// relative precision where it is small.  Both are written here on the hardware's exponential and logarithm (one unit in the
+// last place each): the library forms are three to five times the instructions, and these kernels are bound by them.
 #include "common.h"
 #include <math.h>
 #include <type_traits>
@@ -34,11 +36,33 @@ template <typename F> int by_dtype(int dt, F&& f) {
 
 bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
-__device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
-__device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
+__device__ __forceinline__ float exp_f(float x) { return fast_exp2(1.4426950408889634f * x); }
+
+// ln(1 + e^x).  ln(1 + t) = t * ln(w) / (w - 1) with w the rounded 1 + t: the error of the rounding cancels (Kahan; theorem
+// 4 in Goldberg, "What every computer scientist should know about floating-point arithmetic")
+__device__ __forceinline__ float softplus_f(float x) {
+  const float t = exp_f(x);
+  const float w = 1.0f + t, dw = w - 1.0f;
+  const float l = 0.6931471805599453f * __builtin_amdgcn_logf(w) * (t * __builtin_amdgcn_rcpf(dw));
+  return x > 20.f ? x : (dw == 0.f ? t : l);
+}
+
+// 1 - e^y for y <= 0: the Taylor polynomial up to y^8 on [-1/2, 0] (the next term is below 2^-27 of the result there), else
+// the difference itself (it cannot lose more than two bits)
+__device__ __forceinline__ float one_minus_exp(float y) {
+  float p = 1.f + y * (1.f / 8.f);
+  p = 1.f + y * (1.f / 7.f) * p;
+  p = 1.f + y * (1.f / 6.f) * p;
+  p = 1.f + y * (1.f / 5.f) * p;
+  p = 1.f + y * (1.f / 4.f) * p;
+  p = 1.f + y * (1.f / 3.f) * p;
+  p = 1.f + y * (1.f / 2.f) * p;
+  return y > -0.5f ? -y * p : 1.f - exp_f(y);
+}
+
 // 0.5 (1 + tanh(y)) = sigmoid(2 y)
 __device__ __forceinline__ float gelu_tanh_f(float z) {
-  return z * sigmoid_f(1.5957691216057308f * (z + 0.044715f * z * z * z));
+  return z * fast_sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
 
 // ------------------------------------------------------------------------------------------------ selective scan
@@ -103,27 +127,31 @@ __global__ __launch_bounds__(256) void channel_scan_kernel(ScanArgs a) {
   const T* bp = (const T*)a.bc + (long)q0 * a.bc_stride;
   const T* gp = a.gate ? (const T*)a.gate + (long)q0 * a.gate_stride + col0 : nullptr;
   T* op = (T*)a.out + (long)q0 * a.C + col0;
-  float pu[NU], pd[NU], pb[NQ], pc[NQ];
-  auto fetch = [&](int r0) {                   // this thread's share of a chunk, global -> registers
+  // per staged value: the channel's step bias and skip weight (channel k0 in every pass, CB divides 256)
+  const int k0 = tid & (CB - 1);
+  const bool k_ok = col0 + k0 < a.C;
+  const int kc = k_ok ? k0 : a.C - 1 - col0;
+  // A thread's share of the next chunk, raw: every load is unconditional (rows, channels and states past the end read the
+  // last one there is and are not used), so nothing waits for it before it is stashed a chunk later
+  T pu[NU], pz[NU], pb[NQ], pc[NQ];
+  TD pd[NU];
+  auto fetch = [&](int r0) {
 #pragma unroll
     for (int e = 0; e < NU; ++e) {
-      const int idx = tid + e * 256, t = idx / CB, k = idx & (CB - 1);
-      const bool ok = t < CH && r0 + t < n && col0 + k < a.C;
-      pu[e] = ok ? ldf(up + (long)(r0 + t) * a.u_stride + k) : 0.f;
-      pd[e] = ok ? ldf(dp + (long)(r0 + t) * a.dt_stride + k) : 0.f;
+      const long r = min(r0 + (tid + e * 256) / CB, n - 1);
+      pu[e] = up[r * a.u_stride + kc];
+      pd[e] = dp[r * a.dt_stride + kc];
+      if (gp != nullptr) pz[e] = gp[r * a.gate_stride + kc];
     }
 #pragma unroll
     for (int e = 0; e < NQ; ++e) {
-      const int idx = tid + e * 256, t = idx / NP, j = idx & (NP - 1);
-      const bool ok = t < CH && r0 + t < n && j < a.N;
-      pb[e] = ok ? ldf(bp + (long)(r0 + t) * a.bc_stride + j) : 0.f;
-      pc[e] = ok ? ldf(bp + (long)(r0 + t) * a.bc_stride + a.N + j) : 0.f;
+      const int idx = tid + e * 256, j = min(idx & (NP - 1), a.N - 1);
+      const T* row = bp + min(r0 + idx / NP, n - 1) * a.bc_stride;
+      pb[e] = row[j];
+      pc[e] = row[a.N + j];
     }
   };
   fetch(0);
-  // per staged value: the channel's step bias and skip weight (k = tid & (CB - 1) in every pass, CB divides 256)
-  const int k0 = tid & (CB - 1);
-  const bool k_ok = col0 + k0 < a.C;
   const float bias = a.dt_bias && k_ok ? a.dt_bias[col0 + k0] : 0.f;
   const float skip = a.d_skip && k_ok ? a.d_skip[col0 + k0] : 0.f;
 #pragma unroll
@@ -132,25 +160,27 @@ __global__ __launch_bounds__(256) void channel_scan_kernel(ScanArgs a) {
     float cu[NU], cz[NU];
 #pragma unroll
     for (int e = 0; e < NU; ++e) {
-      const int idx = tid + e * 256, t = idx / CB;
-      cu[e] = pu[e];
+      const int t = (tid + e * 256) / CB;
+      cu[e] = (float)pu[e];
+      cz[e] = gp != nullptr ? fast_silu((float)pz[e]) : 1.f;
       if (t < CH) {
-        const float d = softplus_f(pd[e] + bias);
+        const float d = softplus_f((float)pd[e] + bias);
         sd[t][k0] = d;
-        sdu[t][k0] = d * pu[e];
+        sdu[t][k0] = d * cu[e];
       }
-      cz[e] = gp != nullptr && t < CH && r0 + t < n && k_ok ? ldf(gp + (long)(r0 + t) * a.gate_stride + k0) : 0.f;
     }
 #pragma unroll
     for (int e = 0; e < NQ; ++e) {
       const int idx = tid + e * 256, t = idx / NP, j = idx & (NP - 1);
-      if (t < CH) { sb[t][j] = pb[e]; sc[t][j] = pc[e]; }
+      if (t < CH) {
+        sb[t][j] = j < a.N ? (float)pb[e] : 0.f;
+        sc[t][j] = j < a.N ? (float)pc[e] : 0.f;
+      }
     }
     if (r0 + CH < n) fetch(r0 + CH);
     __syncthreads();
     const int rows = min(CH, n - r0);
-#pragma unroll 2
-    for (int t = 0; t < rows; ++t) {
+    auto row = [&](int t) {
       const float d = sd[t][lc], du = sdu[t][lc];
       float y0 = 0.f, y1 = 0.f;                // (two chains: the sums do not wait for each other)
       if constexpr (R % 4 == 0) {
@@ -172,16 +202,18 @@ __global__ __launch_bounds__(256) void channel_scan_kernel(ScanArgs a) {
       }
       const float y = parts_sum<P, true>(y0 + y1);
       if (part == 0) sy[t][lc] = y;
+    };
+    if (rows == CH) {
+#pragma unroll (CH < 4 ? CH : 4)
+      for (int t = 0; t < CH; ++t) row(t);
+    } else {
+      for (int t = 0; t < rows; ++t) row(t);
     }
     __syncthreads();
 #pragma unroll
     for (int e = 0; e < NU; ++e) {
       const int idx = tid + e * 256, t = idx / CB;
-      if (t < rows && k_ok) {
-        float y = sy[t][k0] + skip * cu[e];
-        if (gp != nullptr) y *= cz[e] * sigmoid_f(cz[e]);
-        stf(op + (long)(r0 + t) * a.C + k0, y);
-      }
+      if (t < rows && k_ok) stf(op + (long)(r0 + t) * a.C + k0, (sy[t][k0] + skip * cu[e]) * cz[e]);
     }
   }
   if (!c_ok) return;
@@ -215,9 +247,9 @@ struct GateArgs {
 
 // one channel's gates from the two products (biases already added) and its input
 __device__ __forceinline__ void unit_gates(float zr, float zi, float rate, float u, float& a, float& drive) {
-  const float log_a = -rate * sigmoid_f(zr);
-  a = expf(log_a);
-  drive = sqrtf(-expm1f(2.0f * log_a)) * sigmoid_f(zi) * u;
+  const float log_a = -rate * fast_sigmoid(zr);
+  a = exp_f(log_a);
+  drive = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * log_a)) * fast_sigmoid(zi) * u;
 }
 
 // any size and type: a workgroup per (row, block); a thread per output channel in turn
@@ -341,12 +373,14 @@ __global__ __launch_bounds__(64 * NW) void gated_unit_scan_kernel(T* __restrict_
   float* st = state + (long)slots[s] * W + cc;
   float S = seq_lens[s] - n > 0 ? *st : 0.f;                     // the state in front of the chunk, in every wave
   float na[L], nd[L];
-  auto fetch = [&](int r0) {
+  T ng[L];
+  auto fetch = [&](int r0) {                                     // (rows past the end read the last one: no load is conditional)
 #pragma unroll
     for (int i = 0; i < L; ++i) {
-      const int r = r0 + wave * L + i;
-      na[i] = r < n ? ap[(long)r * W] : 1.f;                     // (rows past the end leave the state as it is)
-      nd[i] = r < n ? dp[(long)r * W] : 0.f;
+      const long r = min(r0 + wave * L + i, n - 1);
+      na[i] = ap[r * W];
+      nd[i] = dp[r * W];
+      ng[i] = gp[r * gate_stride];
     }
   };
   fetch(0);
@@ -356,12 +390,12 @@ __global__ __launch_bounds__(64 * NW) void gated_unit_scan_kernel(T* __restrict_
     float P = 1.f, Q = 0.f;
 #pragma unroll
     for (int i = 0; i < L; ++i) {
-      va[i] = na[i];
-      vd[i] = nd[i];
+      const bool live = r0 + wave * L + i < n;
+      va[i] = live ? na[i] : 1.f;                                // (rows past the end leave the state as it is)
+      vd[i] = live ? nd[i] : 0.f;
       P *= va[i];
       Q = va[i] * Q + vd[i];
-      const int r = r0 + wave * L + i;
-      vg[i] = r < n ? ldf(gp + (long)r * gate_stride) : 0.f;
+      vg[i] = gelu_tanh_f((float)ng[i] + gb);
     }
     if (r0 + NW * L < n) fetch(r0 + NW * L);
     if constexpr (NW > 1) {
@@ -385,7 +419,7 @@ __global__ __launch_bounds__(64 * NW) void gated_unit_scan_kernel(T* __restrict_
     for (int i = 0; i < L; ++i) {
       carry = va[i] * carry + vd[i];
       const int r = r0 + wave * L + i;
-      if (r < n && ok) stf(op + (long)r * W, carry * gelu_tanh_f(vg[i] + gb));
+      if (r < n && ok) stf(op + (long)r * W, carry * vg[i]);
     }
   }
   if (wave == 0 && ok) *st = S;
@@ -466,11 +500,11 @@ VDAMD_API int vdamd_block_gates(float* a, float* drive, const void* u, const voi
     if constexpr (!std::is_same_v<TT, float>) {
       if (mfma) {
         const int gx = (W / 32 + 3) / 4;
-        const bool tall = T >= 64 && (long)gx * ((T + 63) / 64) >= 256;       // (four row tiles per wave, or one)
-        const dim3 grid(gx, tall ? (T + 63) / 64 : (T + 15) / 16);
-        if (step && tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 4, true>), grid, dim3(256), 0, stream, p);
+        const bool tall = T >= 32 && (long)gx * ((T + 31) / 32) >= 512;       // (two row tiles per wave, or one)
+        const dim3 grid(gx, tall ? (T + 31) / 32 : (T + 15) / 16);
+        if (step && tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 2, true>), grid, dim3(256), 0, stream, p);
         else if (step) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 1, true>), grid, dim3(256), 0, stream, p);
-        else if (tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 4, false>), grid, dim3(256), 0, stream, p);
+        else if (tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 2, false>), grid, dim3(256), 0, stream, p);
         else hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 1, false>), grid, dim3(256), 0, stream, p);
         return;
       }

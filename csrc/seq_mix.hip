@@ -571,6 +571,79 @@ __global__ __launch_bounds__(256) void short_conv_act_kernel(T* __restrict__ out
   }
 }
 
+// The same for 16-bit types and prompt portions: a thread walks ROWS consecutive rows of its 8 channels and keeps the last
+// TAPS - 1 inputs and the taps in registers, so a row is read once per ROWS instead of once per tap.  A row whose history
+// reaches in front of the sequence's rows of this step (or the first row of the walk) fetches it the ordinary way.
+template <typename T, int TAPS, int ROWS>
+__global__ __launch_bounds__(256) void short_conv_act_rows_kernel(T* __restrict__ out, long out_stride,
+                                                                  const T* __restrict__ x, long x_stride,
+                                                                  const T* __restrict__ w, T* __restrict__ state,
+                                                                  const int* __restrict__ slots,
+                                                                  const int* __restrict__ qsl,
+                                                                  const int* __restrict__ seq_lens,
+                                                                  const int* __restrict__ token_seq,
+                                                                  const int* __restrict__ positions, int rows, int C,
+                                                                  int silu, const float* __restrict__ bias, int residual,
+                                                                  const float* __restrict__ in_bias) {
+  using V8 = typename Vec8<T>::type;
+  constexpr int R = TAPS - 1;
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 8;
+  if (c >= C) return;
+  const int t0 = blockIdx.x * ROWS;
+  V8 wv[TAPS], hist[TAPS];                          // hist[j]: the input taps - 1 - j positions back
+  float b8[8], ib[8];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) wv[j] = ld8<T>(w + (long)j * C + c);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) { b8[e] = bias ? bias[c + e] : 0.f; ib[e] = in_bias ? in_bias[c + e] : 0.f; }
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int t = t0 + i;
+    if (t >= rows) return;                          // (the same for the whole workgroup, as is every branch on t below)
+    const int s = token_seq ? token_seq[t] : t;
+    const int n = qsl[s + 1] - qsl[s], pos = positions[t], chunk_start = seq_lens[s] - n;
+    const bool own_state = n == 1;
+    T* st = state + (long)slots[s] * R * C;
+    if (i == 0 || pos - chunk_start < R) {
+#pragma unroll
+      for (int j = 0; j < R; ++j) {
+        const int back = R - j, p = pos - back;
+        if (p >= chunk_start && p >= 0) hist[j] = ld8<T>(x + (long)(t - back) * x_stride + c);
+        else if (p >= 0) hist[j] = ld8<T>(st + (long)(R - (chunk_start - p)) * C + c);
+        else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) hist[j][e] = (T)0.f;
+        }
+      }
+    }
+    hist[R] = ld8<T>(x + (long)t * x_stride + c);
+    if (own_state) {
+#pragma unroll
+      for (int j = 1; j < TAPS; ++j) st8<T>(st + (long)(j - 1) * C + c, hist[j]);
+    }
+    float acc[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[e] = b8[e];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      const bool there = pos - (R - j) >= 0;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[e] += (float)wv[j][e] * ((float)hist[j][e] + (there ? ib[e] : 0.f));
+    }
+    V8 o;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float v = acc[e];
+      if (silu) v = fast_silu(v);
+      if (residual) v += (float)hist[R][e];
+      o[e] = (T)v;
+    }
+    st8<T>(out + (long)t * out_stride + c, o);
+#pragma unroll
+    for (int j = 0; j < R; ++j) hist[j] = hist[j + 1];
+  }
+}
+
 // ---------------------------------------------------------------------------- rotation, head norm, cache write
 struct RotArgs {
   const void* x; long x_stride;             // [T, x_stride]: [q | k | v | ...]
@@ -1322,7 +1395,20 @@ VDAMD_API int vdamd_short_conv_act(void* out, long out_stride, const void* x, lo
     using TT = std::remove_pointer_t<decltype(tp)>;
     bool done = false;
     if constexpr (!std::is_same_v<TT, float>) {
-      if (vec) {
+      // (two rows or more per thread only where that leaves every compute unit several workgroups)
+      const bool walk = vec && taps >= 2 && taps <= 4 && (long)(T / 8) * ((C / 8 + 255) / 256) >= 512;
+      if (walk) {
+        const dim3 grid((T + 7) / 8, (C / 8 + 255) / 256);
+#define CONV_ROWS(TAPS_)                                                                                              \
+  hipLaunchKernelGGL((short_conv_act_rows_kernel<TT, TAPS_, 8>), grid, dim3(256), 0, stream, (TT*)out, out_stride,    \
+                     (const TT*)x, x_stride, (const TT*)conv_w, (TT*)state, slots, qsl, seq_lens, token_seq,          \
+                     positions, T, C, silu, bias, residual, in_bias)
+        if (taps == 4) CONV_ROWS(4);
+        else if (taps == 3) CONV_ROWS(3);
+        else CONV_ROWS(2);
+#undef CONV_ROWS
+        done = true;
+      } else if (vec) {
         hipLaunchKernelGGL((short_conv_act_kernel<TT, true>), dim3(T, (C / 8 + 255) / 256), dim3(256), 0, stream,
                            (TT*)out, out_stride, (const TT*)x, x_stride, (const TT*)conv_w, (TT*)state, slots, qsl,
                            seq_lens, token_seq, positions, C, taps, silu, bias, residual, in_bias);

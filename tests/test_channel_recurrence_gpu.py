@@ -206,3 +206,31 @@ def test_gelu_and_mul(dtype, f):
         for tanh in (True, False):
             want = torch_ref.gelu_and_mul(v, tanh)
             _close(hip.gelu_and_mul(v, tanh), want, dtype, max(1.0, want.abs().max().item()))
+
+
+@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float16])
+@pytest.mark.parametrize("taps", [1, 2, 3, 4, 5])
+def test_convolution_over_many_rows(dtype, taps):
+    """Enough rows that a thread walks several of them: sequences of every short length in between, of which some start
+    and some go on, against the plain form."""
+    hip = _hip()
+    c = 64
+    g = torch.Generator(device="cuda").manual_seed(taps)
+    lens = [1, 2, 1, 3, 4, 5, 1, 1, 7, 8, 9, 31, 2, 600, 1, 3600, 1, 15]
+    ctx = [5, 0, 0, 1, 2, 3, 1, 2, 0, 9, 1, 0, 3, 2, 0, 0, 4, 1]
+    qsl, sls, pos, seq = _batch(lens, ctx)
+    t = sum(lens)
+    x = torch.randn(t, c + 8, device="cuda", generator=g).to(dtype)[:, 8:]
+    w = (torch.randn(taps, c, device="cuda", generator=g) * 0.5).to(dtype)
+    bias, ib = torch.randn(c, device="cuda", generator=g), torch.randn(c, device="cuda", generator=g)
+    slots = torch.randperm(20, device="cuda", generator=g)[:len(lens)].int()
+    st0 = torch.randn(20, max(taps - 1, 1), c, device="cuda", generator=g).to(dtype)
+    for silu, b, res, inb in ((True, bias, False, ib), (False, None, True, None)):
+        s1, s2 = st0.clone(), st0.clone()
+        got = hip.short_conv_act(x, c, w, s1, slots, qsl, sls, seq, pos, silu, True, b, res, inb)
+        want = torch_ref.short_conv_act(x, c, w, s2, slots, qsl, sls, silu, b, res, inb)
+        _close(got, want, dtype, 8)
+        if taps > 1:
+            for i, (n, k) in enumerate(zip(lens, ctx)):            # (rows in front of a sequence's start are never read)
+                seen = min(n + k, taps - 1)
+                assert torch.equal(s1[slots[i], taps - 1 - seen:], s2[slots[i], taps - 1 - seen:]), i
