@@ -275,16 +275,17 @@ __global__ __launch_bounds__(256) void block_gates_kernel(GateArgs p) {
 }
 
 // 16-bit types, n a multiple of 32: a wave owns 32 channels (of one block) x 16 NT rows.  Weights are the A operand, rows
-// of u the B operand, so a lane ends up with 4 neighbouring channels of one row per tile.
-template <typename T, int NT, bool STEP>
+// of u the B operand, so a lane ends up with 4 neighbouring channels of one row per tile.  Of the workgroup's 4 waves, WC
+// lie side by side over channels and 4 / WC over rows: neighbours in either direction share fragments in the CU's cache.
+template <typename T, int NT, int WC, bool STEP>
 __global__ __launch_bounds__(256) void block_gates_mfma_kernel(GateArgs p) {
   using V8 = typename Vec8<T>::type;
   using V4 = typename Vec4<T>::type;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int r16 = lane & 15, g4 = lane >> 4;
-  const int ct = blockIdx.x * (blockDim.x >> 6) + wave;          // 32-channel tile
-  const int row0 = blockIdx.y * 16 * NT;
-  if (ct * 32 >= p.W) return;                                    // (no barrier below: a wave may leave)
+  const int ct = blockIdx.x * WC + wave % WC;                    // 32-channel tile
+  const int row0 = (blockIdx.y * (4 / WC) + wave / WC) * 16 * NT;
+  if (ct * 32 >= p.W || row0 >= p.T) return;                     // (no barrier below: a wave may leave)
   const int n = p.n, b = ct * 32 / n, o0 = ct * 32 - b * n;      // (n % 32 == 0: a tile lies in one block)
   const T* wr = (const T*)p.ra + ((long)b * n + o0 + r16) * n + 8 * g4;
   const T* wi = (const T*)p.ri + ((long)b * n + o0 + r16) * n + 8 * g4;
@@ -441,10 +442,10 @@ VDAMD_API int vdamd_channel_scan(void* out, const void* u, long u_stride, const 
   ScanArgs a{out, u, u_stride, dt, dt_stride, bc, bc_stride, gate, gate_stride, a_log, dt_bias, d_skip, state, slots, qsl,
              seq_lens, C, N};
   const bool step = max_rows == 1;
-  // lanes per channel: as few as hold the states four by four; more where the launch would leave compute units idle
+  // lanes per channel: as few as hold the states four by four; more where the launch would leave a compute unit fewer than two workgroups
   int parts = N <= 16 ? 4 : (N <= 32 ? 8 : 16);
   if (!step)
-    while (parts < 16 && (long)num_seqs * ((C + 256 / parts - 1) / (256 / parts)) < 256) parts <<= 1;
+    while (parts < 16 && (long)num_seqs * ((C + 256 / parts - 1) / (256 / parts)) < 512) parts <<= 1;
   const int r = (N + parts - 1) / parts;
   const dim3 grid((C + 256 / parts - 1) / (256 / parts), num_seqs);
   const int rc = by_dtype(dtype, [&](auto* tp) {
@@ -499,13 +500,13 @@ VDAMD_API int vdamd_block_gates(float* a, float* drive, const void* u, const voi
     using TT = std::remove_pointer_t<decltype(tp)>;
     if constexpr (!std::is_same_v<TT, float>) {
       if (mfma) {
-        const int gx = (W / 32 + 3) / 4;
-        const bool tall = T >= 32 && (long)gx * ((T + 31) / 32) >= 512;       // (two row tiles per wave, or one)
-        const dim3 grid(gx, tall ? (T + 31) / 32 : (T + 15) / 16);
-        if (step && tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 2, true>), grid, dim3(256), 0, stream, p);
-        else if (step) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 1, true>), grid, dim3(256), 0, stream, p);
-        else if (tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 2, false>), grid, dim3(256), 0, stream, p);
-        else hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 1, false>), grid, dim3(256), 0, stream, p);
+        // four row tiles per wave and two by two waves where that leaves every compute unit two workgroups, else one
+        const bool tall = (long)((W / 32 + 1) / 2) * ((T + 127) / 128) >= 512;
+        const dim3 grid = tall ? dim3((W / 32 + 1) / 2, (T + 127) / 128) : dim3((W / 32 + 3) / 4, (T + 15) / 16);
+        if (step && tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 4, 2, true>), grid, dim3(256), 0, stream, p);
+        else if (step) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 1, 4, true>), grid, dim3(256), 0, stream, p);
+        else if (tall) hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 4, 2, false>), grid, dim3(256), 0, stream, p);
+        else hipLaunchKernelGGL((block_gates_mfma_kernel<TT, 1, 4, false>), grid, dim3(256), 0, stream, p);
         return;
       }
     }
