@@ -38,8 +38,8 @@ bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 
 
 __device__ __forceinline__ float exp_f(float x) { return fast_exp2(1.4426950408889634f * x); }
 
-// ln(1 + e^x).  ln(1 + t) = t * ln(w) / (w - 1) with w the rounded 1 + t: the error of the rounding cancels (Kahan; theorem
-// 4 in Goldberg, "What every computer scientist should know about floating-point arithmetic")
+// ln(1 + e^x).  ln(1 + t) = t * ln(w) / (w - 1) with w the rounded 1 + t: the error of the rounding cancels (theorem 4
+// in Goldberg, "What every computer scientist should know about floating-point arithmetic")
 __device__ __forceinline__ float softplus_f(float x) {
   const float t = exp_f(x);
   const float w = 1.0f + t, dw = w - 1.0f;
