@@ -36,17 +36,6 @@ template <typename F> int by_dtype(int dt, F&& f) {
 
 bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
-__device__ __forceinline__ float exp_f(float x) { return fast_exp2(1.4426950408889634f * x); }
-
-// ln(1 + e^x).  ln(1 + t) = t * ln(w) / (w - 1) with w the rounded 1 + t: the error of the rounding cancels (theorem 4
-// in Goldberg, "What every computer scientist should know about floating-point arithmetic")
-__device__ __forceinline__ float softplus_f(float x) {
-  const float t = exp_f(x);
-  const float w = 1.0f + t, dw = w - 1.0f;
-  const float l = 0.6931471805599453f * __builtin_amdgcn_logf(w) * (t * __builtin_amdgcn_rcpf(dw));
-  return x > 20.f ? x : (dw == 0.f ? t : l);
-}
-
 // 1 - e^y for y <= 0: the Taylor polynomial up to y^8 on [-1/2, 0] (the next term is below 2^-27 of the result there), else
 // the difference itself (it cannot lose more than two bits)
 __device__ __forceinline__ float one_minus_exp(float y) {
@@ -57,7 +46,7 @@ __device__ __forceinline__ float one_minus_exp(float y) {
   p = 1.f + y * (1.f / 4.f) * p;
   p = 1.f + y * (1.f / 3.f) * p;
   p = 1.f + y * (1.f / 2.f) * p;
-  return y > -0.5f ? -y * p : 1.f - exp_f(y);
+  return y > -0.5f ? -y * p : 1.f - fast_exp(y);
 }
 
 // 0.5 (1 + tanh(y)) = sigmoid(2 y)
@@ -164,7 +153,7 @@ __global__ __launch_bounds__(256) void channel_scan_kernel(ScanArgs a) {
       cu[e] = (float)pu[e];
       cz[e] = gp != nullptr ? fast_silu((float)pz[e]) : 1.f;
       if (t < CH) {
-        const float d = softplus_f((float)pd[e] + bias);
+        const float d = fast_softplus((float)pd[e] + bias);
         sd[t][k0] = d;
         sdu[t][k0] = d * cu[e];
       }
@@ -248,7 +237,7 @@ struct GateArgs {
 // one channel's gates from the two products (biases already added) and its input
 __device__ __forceinline__ void unit_gates(float zr, float zi, float rate, float u, float& a, float& drive) {
   const float log_a = -rate * fast_sigmoid(zr);
-  a = exp_f(log_a);
+  a = fast_exp(log_a);
   drive = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * log_a)) * fast_sigmoid(zi) * u;
 }
 

@@ -56,6 +56,18 @@ __device__ __forceinline__ float fast_sigmoid(float x) {
 }
 __device__ __forceinline__ float fast_silu(float x) { return x * fast_sigmoid(x); }
 
+__device__ __forceinline__ float fast_exp(float x) { return fast_exp2(1.4426950408889634f * x); }
+
+// ln(1 + e^x), in full relative precision where it is small.  ln(1 + t) = t * ln(w) / (w - 1) with w the rounded 1 + t: the
+// error of the rounding cancels (theorem 4 in Goldberg, "What every computer scientist should know about floating-point
+// arithmetic")
+__device__ __forceinline__ float fast_softplus(float x) {
+  const float t = fast_exp(x);
+  const float w = 1.0f + t, dw = w - 1.0f;
+  const float l = 0.6931471805599453f * __builtin_amdgcn_logf(w) * (t * __builtin_amdgcn_rcpf(dw));
+  return x > 20.f ? x : (dw == 0.f ? t : l);
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);

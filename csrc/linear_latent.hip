@@ -10,10 +10,15 @@
 //                            one head's S for one sequence, in registers (up to 16 waves x dim/16 rows each), and walks
 //                            the sequence's rows in chunks staged through LDS: prompt portions and single decoded rows
 //                            are the same kernel (launches of decoded rows only take small workgroups)
+//   channel_decay_attention  the same recurrence with a decay per row, head and key channel, S <- diag(alpha) S + k v^T.  A
+//                            lane owns two columns, so every q / k / alpha value read from LDS serves two of them
+//   low_rank_decay           sigmoid(a . w[c] + bias[c])^(1 / tau) of rows a of a narrow projection: the products, the bias
+//                            and the decay of a channel in one pass, fp32
 //   gated_rms_norm           o / sqrt(mean(o^2) + eps) * w * sigmoid(g) * scale (or silu(g)), over whole rows or over runs of `group`
 //                            values (heads) that share w
 //   clamped_glu              min(g, L) sigmoid(alpha min(g, L)) (clamp(u, -L, L) + 1) over [g | u]
 //   relu_squared             max(x, 0)^2
+//   weighted_relu_squared    max(w x, 0)^2 of expert-sorted rows, w the routing weight of the row's (token, choice) slot
 //   expert_epilogue          routed + x * (weights of the chosen identity experts) + shared * sigmoid(gate)
 //   latent_prep              per token: RMS norm of the latent and rotation of the shared key part into the row cache;
 //                            the query [q_lat | rotated q_rope] assembled; angles = position * frequency in fp32
@@ -270,6 +275,30 @@ __global__ void relu_squared_kernel(T* __restrict__ out, const T* __restrict__ x
   }
 }
 
+// out[row] = max(w * h[row], 0)^2 for the sorted row of every (token, choice) slot: an expert whose INPUT carries the routing
+// weight (its up projection has no bias, so the weight may as well multiply what comes out of it).  grid (slots)
+template <typename T, int W>
+__global__ __launch_bounds__(256) void weighted_relu_squared_kernel(T* __restrict__ out, const T* __restrict__ h,
+                                                                    long h_stride, const float* __restrict__ topw,
+                                                                    const int* __restrict__ inv, int F) {
+  const long row = inv[blockIdx.x];
+  const float w = topw[blockIdx.x];
+  const T* hr = h + row * h_stride;
+  T* o = out + row * (long)F;
+  for (int i = threadIdx.x * W; i < F; i += blockDim.x * W) {
+    if constexpr (W == 8) {
+      const typename Vec8<T>::type v = ld8<T>(hr + i);
+      typename Vec8<T>::type r;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) { const float f = fmaxf(w * (float)v[e], 0.f); r[e] = (T)(f * f); }
+      st8<T>(o + i, r);
+    } else {
+      const float f = fmaxf(w * ldf(hr + i), 0.f);
+      stf(o + i, f * f);
+    }
+  }
+}
+
 // ------------------------------------------------------------------------------------------------ linear attention
 // grid (sequences, heads, column tiles of 64), G waves: thread (g = tid / 64, c = tid % 64) owns rows
 // g * R .. g * R + R - 1 of column c of the head's state, in registers (G * R >= dim).  x rows hold [q (H * dim) | k (H * dim) |
@@ -374,6 +403,179 @@ __global__ __launch_bounds__(64 * G) __attribute__((amdgpu_waves_per_eu(G >= 16 
       if (r < dim) st[(long)r * vdim + col0 + lane] = S[i];
     }
   }
+}
+
+// A decay per row, head and key channel (alpha [T, H * dim] fp32).  grid (sequences, heads, column tiles of 64), NW waves:
+// lane (half, c) of wave w owns rows (2 w + half) * R .. + R - 1 of columns 2 c and 2 c + 1 of the head's state, in
+// registers.  Rows in chunks of C as above; a chunk's q / k / alpha (the whole head) and v (the tile) are staged in LDS, and
+// each value read back serves two columns.  A step's two column sums meet across the halves of the wave in one lane swap, so
+// a wave leaves 64 partial sums per row.  Loads are unconditional (addresses clamped into the sequence's rows): the next
+// chunk's are in flight while the current one is computed.
+template <typename T, int R, int NW, int C>
+__global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(NW >= 16 ? 8 : 1, 8))) void channel_decay_attention_kernel(
+    float* __restrict__ out, const T* __restrict__ x, long x_stride, const float* __restrict__ alpha,
+    float* __restrict__ state, const int* __restrict__ slots, const int* __restrict__ qsl,
+    const int* __restrict__ seq_lens, int H, int dim, int vdim, float scale, int silu) {
+  constexpr int W = 2 * NW * R, TH = 64 * NW;
+  constexpr int NQ = C * W / TH;
+  constexpr int NV = (C * 64 + TH - 1) / TH;
+  static_assert(R % 4 == 0 && (C * W) % TH == 0, "chunk does not divide over the threads");
+  __shared__ __attribute__((aligned(16))) float qs[C][W];
+  __shared__ __attribute__((aligned(16))) float ks[C][W];
+  __shared__ __attribute__((aligned(16))) float as[C][W];
+  __shared__ __attribute__((aligned(16))) float vs[C][64];
+  __shared__ float part[NW][C][64];
+  const int b = blockIdx.x, h = blockIdx.y;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, half = lane >> 5, cp = lane & 31;
+  const int col0 = blockIdx.z * 64, c0 = col0 + 2 * cp;
+  const int row0 = (2 * wave + half) * R;
+  const int s = qsl[b], e = qsl[b + 1];
+  if (e <= s) return;                                            // (uniform over the workgroup)
+  const bool fresh = seq_lens[b] - (e - s) <= 0;                 // whatever the slot holds is not ours
+  float* st = state + ((long)slots[b] * H + h) * (long)dim * vdim;
+  const bool pair = (vdim & 1) == 0;                             // (both columns of a lane exist or none, 8-byte aligned)
+  float S0[R], S1[R];
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int r = row0 + i;
+    S0[i] = S1[i] = 0.f;
+    if (!fresh && r < dim && c0 < vdim) {
+      const float* p = st + (long)r * vdim + c0;
+      if (pair) { const float2 f = *reinterpret_cast<const float2*>(p); S0[i] = f.x; S1[i] = f.y; }
+      else { S0[i] = p[0]; if (c0 + 1 < vdim) S1[i] = p[1]; }
+    }
+  }
+  const long qoff = (long)h * dim, koff = (long)(H + h) * dim, voff = 2L * H * dim + (long)h * vdim;
+  auto act = [&](float f) { return silu ? f * sigmoid_f(f) : f; };
+  T pq[NQ], pk[NQ], pv[NV];
+  float pa[NQ];
+  auto fetch = [&](int r0) {
+#pragma unroll
+    for (int u = 0; u < NQ; ++u) {
+      const int idx = tid + TH * u, t = idx / W, j = min(idx - t * W, dim - 1);
+      const long row = min(r0 + t, e - 1);
+      const T* xr = x + row * x_stride;
+      pq[u] = xr[qoff + j];
+      pk[u] = xr[koff + j];
+      pa[u] = alpha[(row * H + h) * (long)dim + j];
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int idx = tid + TH * u, t = min(idx >> 6, C - 1), c = min(col0 + (idx & 63), vdim - 1);
+      pv[u] = x[(long)min(r0 + t, e - 1) * x_stride + voff + c];
+    }
+  };
+  fetch(s);
+  for (int r0 = s; r0 < e; r0 += C) {
+    const int n = min(C, e - r0);
+#pragma unroll
+    for (int u = 0; u < NQ; ++u) {
+      const int idx = tid + TH * u, t = idx / W, j = idx - t * W;
+      const bool in = j < dim;                                   // (rows past dim stay zero: no key, nothing to decay)
+      qs[t][j] = in ? act((float)pq[u]) : 0.f;
+      ks[t][j] = in ? act((float)pk[u]) : 0.f;
+      as[t][j] = pa[u];
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int idx = tid + TH * u;
+      if (idx < C * 64) vs[idx >> 6][idx & 63] = act((float)pv[u]);
+    }
+    if (r0 + C < e) fetch(r0 + C);
+    __syncthreads();
+#pragma unroll 2
+    for (int t = 0; t < n; ++t) {
+      const float2 v = *reinterpret_cast<const float2*>(&vs[t][2 * cp]);
+      const f32x4* k4 = reinterpret_cast<const f32x4*>(&ks[t][row0]);
+      const f32x4* q4 = reinterpret_cast<const f32x4*>(&qs[t][row0]);
+      const f32x4* d4 = reinterpret_cast<const f32x4*>(&as[t][row0]);
+      float a0 = 0.f, a1 = 0.f, b0 = 0.f, b1 = 0.f;              // (two chains per column)
+#pragma unroll
+      for (int i = 0; i < R / 4; ++i) {
+        const f32x4 kk = k4[i], qq = q4[i], dd = d4[i];
+#pragma unroll
+        for (int u = 0; u < 4; u += 2) {
+          const int m = 4 * i + u;
+          S0[m] = dd[u] * S0[m] + kk[u] * v.x;                 a0 += S0[m] * qq[u];
+          S1[m] = dd[u] * S1[m] + kk[u] * v.y;                 a1 += S1[m] * qq[u];
+          S0[m + 1] = dd[u + 1] * S0[m + 1] + kk[u + 1] * v.x; b0 += S0[m + 1] * qq[u + 1];
+          S1[m + 1] = dd[u + 1] * S1[m + 1] + kk[u + 1] * v.y; b1 += S1[m + 1] * qq[u + 1];
+        }
+      }
+      // lanes 0 .. 31 end up with both halves' sums of column 2 cp, the others with those of column 2 cp + 1
+      const auto sw = __builtin_amdgcn_permlane32_swap(__float_as_uint(a0 + b0), __float_as_uint(a1 + b1), false, false);
+      part[wave][t][2 * cp + half] = __uint_as_float(sw[0]) + __uint_as_float(sw[1]);
+    }
+    __syncthreads();
+    for (int idx = tid; idx < n * 64; idx += TH) {
+      const int t = idx >> 6, c = idx & 63;
+      if (col0 + c < vdim) {
+        float sum = 0.f;
+#pragma unroll
+        for (int w = 0; w < NW; ++w) sum += part[w][t][c];
+        out[(long)(r0 + t) * H * vdim + (long)h * vdim + col0 + c] = sum * scale;
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int r = row0 + i;
+    if (r < dim && c0 < vdim) {
+      float* p = st + (long)r * vdim + c0;
+      if (pair) *reinterpret_cast<float2*>(p) = make_float2(S0[i], S1[i]);
+      else { p[0] = S0[i]; if (c0 + 1 < vdim) p[1] = S1[i]; }
+    }
+  }
+}
+
+// grid (channel tiles of 256, row tiles of ROWS): a thread owns one channel for ROWS rows; the rows' narrow vectors are
+// staged 32 values at a time, a channel's weights are read once for all of them.
+// alpha = sigmoid(z)^(1 / tau) = exp(-softplus(-z) / tau), z = a . w[c] + bias[c]
+template <typename T, int ROWS>
+__global__ __launch_bounds__(256) void low_rank_decay_kernel(float* __restrict__ out, const T* __restrict__ a, long a_stride,
+                                                             const T* __restrict__ w, const float* __restrict__ bias, int rows,
+                                                             int C, int rank, float inv_tau) {
+  __shared__ __attribute__((aligned(16))) float xs[ROWS][32];
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  const int t0 = blockIdx.y * ROWS;
+  const T* wr = w + (long)min(c, C - 1) * rank;
+  float acc[ROWS];
+#pragma unroll
+  for (int t = 0; t < ROWS; ++t) acc[t] = 0.f;
+  const bool vec = rank % 8 == 0 && !std::is_same_v<T, float>;
+  for (int j0 = 0; j0 < rank; j0 += 32) {
+    __syncthreads();
+    for (int i = threadIdx.x; i < ROWS * 32; i += 256) {
+      const int t = i >> 5, j = j0 + (i & 31);
+      xs[t][i & 31] = j < rank ? ldf(a + (long)min(t0 + t, rows - 1) * a_stride + j) : 0.f;
+    }
+    __syncthreads();
+    const int n = min(32, rank - j0);
+    for (int j = 0; j < n; j += 8) {
+      float wv[8];
+      if (vec) {
+        if constexpr (!std::is_same_v<T, float>) {
+          const typename Vec8<T>::type v = ld8<T>(wr + j0 + j);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) wv[e] = (float)v[e];
+        }
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) wv[e] = j + e < n ? ldf(wr + j0 + j + e) : 0.f;
+      }
+#pragma unroll
+      for (int t = 0; t < ROWS; ++t) {
+        const f32x4 x0 = *reinterpret_cast<const f32x4*>(&xs[t][j]), x1 = *reinterpret_cast<const f32x4*>(&xs[t][j + 4]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[t] += wv[e] * x0[e] + wv[e + 4] * x1[e];
+      }
+    }
+  }
+  if (c >= C) return;
+  const float bc = bias != nullptr ? bias[c] : 0.f;
+#pragma unroll
+  for (int t = 0; t < ROWS; ++t)
+    if (t0 + t < rows) out[(long)(t0 + t) * C + c] = fast_exp(-fast_softplus(-(acc[t] + bc)) * inv_tau);
 }
 
 // ------------------------------------------------------------------------------------------------ latent attention
@@ -727,6 +929,82 @@ VDAMD_API int vdamd_decay_linear_attention(float* out, const void* x, long x_str
       else DLA(16, 16, 8);
     }
 #undef DLA
+  });
+  if (rc) return 1;
+  HIP_LAUNCH_CHECK();
+  return 0;
+}
+
+// the same with a decay per row, head and key channel, alpha [T, H * dim] fp32; out = scale * S^T q
+VDAMD_API int vdamd_channel_decay_attention(float* out, const void* x, long x_stride, const float* alpha, float* state,
+                                            const int* slots, const int* qsl, const int* seq_lens, int num_seqs, int H,
+                                            int dim, int vdim, float scale, int silu, int max_rows, int dt,
+                                            hipStream_t stream) {
+  if (num_seqs <= 0) return 0;
+  if (H <= 0 || dim <= 0 || vdim <= 0 || dim > 256) return 1;
+  const dim3 grid(num_seqs, H, (vdim + 63) / 64);
+  const int rc = by_dtype(dt, [&](auto* tp) {
+    using TT = std::remove_pointer_t<decltype(tp)>;
+#define CDA(R_, NW_, C_)                                                                                              \
+  hipLaunchKernelGGL((channel_decay_attention_kernel<TT, R_, NW_, C_>), grid, dim3(64 * NW_), 0, stream, out,          \
+                     (const TT*)x, x_stride, alpha, state, slots, qsl, seq_lens, H, dim, vdim, scale, silu)
+    if (max_rows > 0 && max_rows <= 2) {                         // decoded rows: bound by the states, small workgroups
+      if (dim <= 32) CDA(4, 4, 8);
+      else if (dim <= 64) CDA(8, 4, 4);
+      else if (dim <= 128) CDA(16, 4, 4);
+      else CDA(32, 4, 4);
+    } else {                                                     // prompt portions: bound by the walk over the rows
+      if (dim <= 32) CDA(4, 4, 8);
+      else if (dim <= 64) CDA(4, 8, 8);
+      else if (dim <= 128) CDA(4, 16, 8);
+      else CDA(8, 16, 8);
+    }
+#undef CDA
+  });
+  if (rc) return 1;
+  HIP_LAUNCH_CHECK();
+  return 0;
+}
+
+// a [rows, rank] (row stride a_stride), w [C, rank] of type dt, bias [C] fp32 or null -> out [rows, C] fp32
+VDAMD_API int vdamd_low_rank_decay(float* out, const void* a, long a_stride, const void* w, const float* bias, int rows, int C,
+                                   int rank, float inv_tau, int dt, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  if (C <= 0 || rank <= 0) return 1;
+  const int rc = by_dtype(dt, [&](auto* tp) {
+    using TT = std::remove_pointer_t<decltype(tp)>;
+    if (rows >= 1024)
+      hipLaunchKernelGGL((low_rank_decay_kernel<TT, 16>), dim3((C + 255) / 256, (rows + 15) / 16), dim3(256), 0, stream, out,
+                         (const TT*)a, a_stride, (const TT*)w, bias, rows, C, rank, inv_tau);
+    else
+      hipLaunchKernelGGL((low_rank_decay_kernel<TT, 4>), dim3((C + 255) / 256, (rows + 3) / 4), dim3(256), 0, stream, out,
+                         (const TT*)a, a_stride, (const TT*)w, bias, rows, C, rank, inv_tau);
+  });
+  if (rc) return 1;
+  HIP_LAUNCH_CHECK();
+  return 0;
+}
+
+// h [rows, F] (row stride h_stride) expert-sorted, inv [slots] the row of every slot, topw [slots]; rows of no slot stay as they are
+VDAMD_API int vdamd_weighted_relu_squared(void* out, const void* h, long h_stride, const float* topw, const int* inv, int slots,
+                                          int F, int dt, hipStream_t stream) {
+  if (slots <= 0) return 0;
+  if (F <= 0) return 1;
+  const bool vec = dt != DT_F32 && F % 8 == 0 && h_stride % 8 == 0 && aligned16(h) && aligned16(out);
+  const int threads = (vec ? F / 8 : F) >= 256 ? 256 : ((vec ? F / 8 : F) >= 128 ? 128 : 64);
+  const int rc = by_dtype(dt, [&](auto* tp) {
+    using TT = std::remove_pointer_t<decltype(tp)>;
+    bool done = false;
+    if constexpr (!std::is_same_v<TT, float>) {
+      if (vec) {
+        hipLaunchKernelGGL((weighted_relu_squared_kernel<TT, 8>), dim3(slots), dim3(threads), 0, stream, (TT*)out,
+                           (const TT*)h, h_stride, topw, inv, F);
+        done = true;
+      }
+    }
+    if (!done)
+      hipLaunchKernelGGL((weighted_relu_squared_kernel<TT, 1>), dim3(slots), dim3(threads), 0, stream, (TT*)out, (const TT*)h,
+                         h_stride, topw, inv, F);
   });
   if (rc) return 1;
   HIP_LAUNCH_CHECK();

@@ -400,7 +400,7 @@ __global__ __launch_bounds__(ALIGN_THREADS) void moe_route_small_kernel(
   }
 }
 
-// grid (token, 2048-column slab); y rows are in expert-sorted order
+// grid (token, 2048-column slab); y rows are in expert-sorted order; topw null: every weight is one
 template <typename T>
 __global__ __launch_bounds__(256) void moe_combine_kernel(T* __restrict__ out, long out_stride,
                                                           const T* __restrict__ y, long y_stride,
@@ -417,7 +417,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(T* __restrict__ out, l
   if (threadIdx.x < k) {
     const int e = topi[(long)t * k + threadIdx.x];
     const bool local = local_experts < 0 || (e >= expert_start && e < expert_start + local_experts);
-    w[threadIdx.x] = local ? topw[(long)t * k + threadIdx.x] : 0.f;
+    w[threadIdx.x] = !local ? 0.f : (topw != nullptr ? topw[(long)t * k + threadIdx.x] : 1.f);
     pos[threadIdx.x] = local ? inv[(long)t * k + threadIdx.x] : -1;
     loc[threadIdx.x] = e - expert_start;
   }

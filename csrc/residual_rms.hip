@@ -4,6 +4,7 @@
 //   residual_rms     one launch per sublayer boundary.  With x the fp32 residual stream (updated in place):
 //                      x += a + b                      (outputs of two sublayers that read the same input; either absent)
 //                      x += y / rms(y) * post_w * post_scale (an output RMS-normed before it joins the stream; absent)
+//                      x += z / rms(z) * post_w2 * post_scale (a second one of the kind; absent)
 //                      out = x / rms(x) * (offset + w) (the next sublayer's input) or out = x, in any float type
 //                    and, with nothing to add, the plain RMS norm of rows of any float type (fp32 gains)
 //   gelu_mul_rows    gelu_tanh(g[t, :]) * table[ids[t], col : col + n]
@@ -66,11 +67,13 @@ struct ResidualArgs {
   const void* a; long a_stride;      // [rows, H] or null
   const void* b; long b_stride;      // [rows, H] or null
   const void* y; long y_stride;      // [rows, H] or null
+  const void* z; long z_stride;      // [rows, H] or null (only with y)
   const float* post_w;               // [H] (with y)
+  const float* post_w2;              // [H] (with z)
   const float* w;                    // [H] or null: no gain
   float offset, eps;
   int H, normed;
-  float post_scale;                  // (with y)
+  float post_scale;                  // (with y and z)
 };
 
 // W values per thread and turn (4: rows whose length, strides and addresses allow 16 / 8-byte accesses).  A row is
@@ -83,16 +86,17 @@ __global__ void residual_rms_kernel(ResidualArgs p) {
   const TA* ar = p.a ? (const TA*)p.a + row * p.a_stride : nullptr;
   const TA* br = p.b ? (const TA*)p.b + row * p.b_stride : nullptr;
   const TA* yr = p.y ? (const TA*)p.y + row * p.y_stride : nullptr;
+  const TA* zr = p.z ? (const TA*)p.z + row * p.z_stride : nullptr;
   const int n = p.H / W;
-  float inv_y = 0.f;
-  if (yr != nullptr) {
+  auto inv_rms = [&](const TA* r) {                 // post_scale / rms of a row
     float ss = 0.f;
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
-      if constexpr (W == 4) { const f32x4 v = ld4<TA>(yr + 4 * i); ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
-      else { const float v = ldf(yr + i); ss += v * v; }
+      if constexpr (W == 4) { const f32x4 v = ld4<TA>(r + 4 * i); ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
+      else { const float v = ldf(r + i); ss += v * v; }
     }
-    inv_y = p.post_scale / sqrtf(block_sum(ss, red) / (float)p.H + p.eps);
-  }
+    return p.post_scale / sqrtf(block_sum(ss, red) / (float)p.H + p.eps);
+  };
+  const float inv_y = yr != nullptr ? inv_rms(yr) : 0.f, inv_z = zr != nullptr ? inv_rms(zr) : 0.f;
   const bool adds = ar != nullptr || yr != nullptr;
   float ss = 0.f;
   for (int i = threadIdx.x; i < n; i += blockDim.x) {
@@ -109,6 +113,10 @@ __global__ void residual_rms_kernel(ResidualArgs p) {
             const f32x4 yv = ld4<TA>(yr + 4 * i), pw = *reinterpret_cast<const f32x4*>(p.post_w + 4 * i);
             r += yv * inv_y * pw;
           }
+          if (zr != nullptr) {
+            const f32x4 zv = ld4<TA>(zr + 4 * i), pw = *reinterpret_cast<const f32x4*>(p.post_w2 + 4 * i);
+            r += zv * inv_z * pw;
+          }
           *reinterpret_cast<f32x4*>(xr + 4 * i) = r;
         }
       }
@@ -119,6 +127,7 @@ __global__ void residual_rms_kernel(ResidualArgs p) {
         if (adds) {
           if (ar != nullptr) r += br != nullptr ? ldf(ar + i) + ldf(br + i) : ldf(ar + i);
           if (yr != nullptr) r += ldf(yr + i) * inv_y * p.post_w[i];
+          if (zr != nullptr) r += ldf(zr + i) * inv_z * p.post_w2[i];
           xr[i] = r;
         }
       }
@@ -221,16 +230,18 @@ __global__ void gelu_and_mul_kernel(T* __restrict__ out, const T* __restrict__ x
 // x_dt: the type of x (DT_F32 whenever a / b / y is given: x is then the residual stream, updated in place);
 // in_dt: the type of a, b and y; out_dt: the type of out.  normed 0: out = x (after the adds).
 VDAMD_API int vdamd_residual_rms(void* out, long out_stride, void* x, long x_stride, const void* a, long a_stride,
-                                 const void* b, long b_stride, const void* y, long y_stride, const float* post_w,
-                                 const float* w, float offset, float eps, int rows, int H, int normed, int x_dt,
+                                 const void* b, long b_stride, const void* y, long y_stride, const void* z,
+                                 long z_stride, const float* post_w, const float* post_w2, const float* w, float offset, float eps, int rows, int H, int normed, int x_dt,
                                  int in_dt, int out_dt, float post_scale, hipStream_t stream) {
   if (rows <= 0) return 0;
-  if (H <= 0 || (b != nullptr && a == nullptr) || (y != nullptr && post_w == nullptr)) return 1;
+  if (H <= 0 || (b != nullptr && a == nullptr) || (y != nullptr && post_w == nullptr) ||
+      (z != nullptr && (y == nullptr || post_w2 == nullptr)))
+    return 1;
   if ((a != nullptr || y != nullptr) && x_dt != DT_F32) return 1;
-  ResidualArgs p{out, out_stride, x, x_stride, a, a_stride, b, b_stride, y, y_stride, post_w, w, offset, eps, H, normed,
-                 post_scale};
+  ResidualArgs p{out, out_stride, x, x_stride, a, a_stride, b, b_stride, y, y_stride, z, z_stride, post_w, post_w2, w, offset, eps,
+                 H, normed, post_scale};
   const bool vec = H % 4 == 0 && x_stride % 4 == 0 && out_stride % 4 == 0 && a_stride % 4 == 0 && b_stride % 4 == 0 &&
-                   y_stride % 4 == 0 && aligned16(x) && aligned16(out) && aligned16(a) && aligned16(b) &&
+                   y_stride % 4 == 0 && z_stride % 4 == 0 && aligned16(z) && aligned16(post_w2) && aligned16(x) && aligned16(out) && aligned16(a) && aligned16(b) &&
                    aligned16(y) && aligned16(w) && aligned16(post_w);
   const dim3 grid(rows), block(row_threads(vec ? H : 4 * H));
   int r1 = 0, r2 = 0;

@@ -650,11 +650,13 @@ struct RotArgs {
   const float* inv_freq; int half;          // [half] angular frequencies
   float rot_scale, eps;                     // factor on cos and sin
   const float* q_norm; const float* k_norm; // [D] or null
+  const float* bias;                        // [H * D + G * D + G * Dv] or null: added to x first
   const int* positions;                     // [T]
   void* q_out;                              // [T, H, D]
   void* k_cache; void* v_cache;             // [blocks, G, bs, D], [blocks, G, bs / 8, Dv, 8] or null
   const int* slot_mapping;                  // [T]
   int H, G, D, Dv, bs, interleaved;
+  int normed;                               // 0: no head norm (q and k as they are, biased and rotated)
 };
 
 constexpr int ROT_MAX_HALF = 256;
@@ -681,6 +683,7 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_kernel(RotArgs a) {
   const int off = slot >= 0 ? slot % a.bs : 0;
   for (int u = wave; u < a.H + a.G; u += nwaves) {
     const T* src = xr + (long)u * a.D;
+    const float* b = a.bias ? a.bias + (long)u * a.D : nullptr;
     float v[UNIT_MAX_PER_LANE];
     float ss = 0.f;
 #pragma unroll
@@ -688,17 +691,17 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_kernel(RotArgs a) {
       const int d = lane + it * 64;
       v[it] = 0.f;
       if (d >= a.D) continue;
-      v[it] = ldf(src + d);
+      v[it] = ldf(src + d) + (b ? b[d] : 0.f);
       if (d < 2 * a.half) {
         const int i = a.interleaved ? d >> 1 : (d < a.half ? d : d - a.half);
         const bool second = a.interleaved ? (d & 1) : d >= a.half;
         const int pd = a.interleaved ? d ^ 1 : (second ? d - a.half : d + a.half);
-        const float o = ldf(src + pd);
+        const float o = ldf(src + pd) + (b ? b[pd] : 0.f);
         v[it] = second ? v[it] * cs[i] + o * sn[i] : v[it] * cs[i] - o * sn[i];
       }
       ss += v[it] * v[it];
     }
-    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.D + a.eps);
+    const float inv = a.normed ? 1.0f / sqrtf(wave_sum(ss) / (float)a.D + a.eps) : 1.f;
     const bool is_q = u < a.H;
     const float* w = is_q ? a.q_norm : a.k_norm;
     if (!is_q && slot < 0) continue;
@@ -712,9 +715,11 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_kernel(RotArgs a) {
   }
   if (slot < 0) return;
   const T* vr = xr + (long)(a.H + a.G) * a.D;
+  const float* vb = a.bias ? a.bias + (long)(a.H + a.G) * a.D : nullptr;
   for (int i = threadIdx.x; i < a.G * a.Dv; i += blockDim.x) {
     const int g = i / a.Dv, d = i - g * a.Dv;
-    ((T*)a.v_cache)[(((blk * a.G + g) * (a.bs >> 3) + (off >> 3)) * (long)a.Dv + d) * 8 + (off & 7)] = vr[i];
+    ((T*)a.v_cache)[(((blk * a.G + g) * (a.bs >> 3) + (off >> 3)) * (long)a.Dv + d) * 8 + (off & 7)] =
+        vb ? (T)(ldf(vr + i) + vb[i]) : vr[i];
   }
 }
 
@@ -735,20 +740,24 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_vec_kernel(RotArgs a, i
   for (int idx = threadIdx.x; idx < (a.H + a.G) * L; idx += blockDim.x) {
     const int u = idx >> sh, d = (idx & (L - 1)) * 8;
     const V8 xv = ld8<T>(xr + (long)u * a.D + d);
+    const float* b = a.bias ? a.bias + (long)u * a.D + d : nullptr;
     float v[8];
     float ss = 0.f;
 #pragma unroll
     for (int e = 0; e < 8; e += 2) {
       const int i = (d + e) >> 1;
-      const float p = (float)xv[e], q = (float)xv[e + 1];
+      const float p = (float)xv[e] + (b ? b[e] : 0.f), q = (float)xv[e + 1] + (b ? b[e + 1] : 0.f);
       const bool rot = i < a.half;
       const float c = rot ? cs[i] : 1.f, s = rot ? sn[i] : 0.f;
       v[e] = p * c - q * s;
       v[e + 1] = q * c + p * s;
       ss += v[e] * v[e] + v[e + 1] * v[e + 1];
     }
-    for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
-    const float inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+    float inv = 1.f;
+    if (a.normed) {
+      for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
+      inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+    }
     const bool is_q = u < a.H;
     const float* w = is_q ? a.q_norm : a.k_norm;
     V8 r;
@@ -761,7 +770,12 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_vec_kernel(RotArgs a, i
   const T* vr = xr + (long)(a.H + a.G) * a.D;
   for (int i = threadIdx.x * 8; i < a.G * a.Dv; i += blockDim.x * 8) {
     const int g = i / a.Dv, d = i - g * a.Dv;                     // (Dv % 8 == 0: the 8 channels share a head)
-    const V8 vv = ld8<T>(vr + i);
+    V8 vv = ld8<T>(vr + i);
+    if (a.bias) {
+      const float* vb = a.bias + (long)(a.H + a.G) * a.D + i;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) vv[e] = (T)((float)vv[e] + vb[e]);
+    }
     T* vd = (T*)a.v_cache + (((blk * a.G + g) * (a.bs >> 3) + (off >> 3)) * (long)a.Dv + d) * 8 + (off & 7);
 #pragma unroll
     for (int e = 0; e < 8; ++e) vd[e * 8] = vv[e];
@@ -1348,19 +1362,20 @@ VDAMD_API int vdamd_conv_norm_cache(const void* x, long x_stride, const void* co
 }
 
 // x [T, x_stride] = [q (H * D) | k (G * D) | v (G * Dv)], q_out [T, H, D]; caches may be null (nothing is written then).
-// inv_freq [half] (null with half 0), 2 half <= D <= 512; interleaved: neighbours are paired, else values half apart
+// inv_freq [half] (null with half 0), 2 half <= D <= 512; interleaved: neighbours are paired, else values half apart.
+// bias [columns of q, k and v] or null joins x first; normed 0: no head norm.  G may be 0 (queries only)
 VDAMD_API int vdamd_rotate_norm_cache(void* q_out, const void* x, long x_stride, const float* inv_freq, int half,
                                       float rot_scale, int interleaved, float eps, const float* q_norm,
-                                      const float* k_norm, const int* positions, void* k_cache, void* v_cache,
-                                      const int* slot_mapping, int T, int H, int G, int D, int Dv, int bs, int dt,
-                                      hipStream_t stream) {
+                                      const float* k_norm, const float* bias, const int* positions, void* k_cache,
+                                      void* v_cache, const int* slot_mapping, int T, int H, int G, int D, int Dv, int bs,
+                                      int normed, int dt, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (H <= 0 || G <= 0 || H % G || D <= 0 || D > 64 * UNIT_MAX_PER_LANE || Dv <= 0 || half < 0 || 2 * half > D ||
+  if (H <= 0 || G < 0 || (G > 0 && H % G) || (G == 0 && k_cache != nullptr) || D <= 0 || D > 64 * UNIT_MAX_PER_LANE || Dv <= 0 || half < 0 || 2 * half > D ||
       half > ROT_MAX_HALF || (half > 0 && inv_freq == nullptr))
     return 1;
   if (k_cache != nullptr && (v_cache == nullptr || slot_mapping == nullptr || bs <= 0 || bs % 8)) return 1;
-  RotArgs a{x, x_stride, inv_freq, half, rot_scale, eps, q_norm, k_norm, positions, q_out, k_cache, v_cache, slot_mapping,
-            H, G, D, Dv, bs, interleaved};
+  RotArgs a{x, x_stride, inv_freq, half, rot_scale, eps, q_norm, k_norm, bias, positions, q_out, k_cache, v_cache,
+            slot_mapping, H, G, D, Dv, bs, interleaved, normed};
   const int L = D / 8;
   auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
   const bool vec = dt != DT_F32 && (interleaved || half == 0) && D % 8 == 0 && (L & (L - 1)) == 0 && L <= 64 &&

@@ -106,6 +106,9 @@ class Attention(nn.Module):
         self.scale = scale
         # a query sees its last `window` keys only (0 = the whole context)
         self.window = int(sliding_window or 0)
+        # how far back ANY reader of this layer's cache looks (0 = the whole context): layers that share keys and values
+        # may be masked otherwise than the layer that owns them
+        self.reach = self.window
         # scores squashed to softcap * tanh(score / softcap) before the softmax (Gemma-2); 0 = off
         self.softcap = float(softcap or 0.0)
         self.layer_idx = layer_idx
@@ -120,6 +123,10 @@ class Attention(nn.Module):
 
     def bind_kv_cache(self, k_cache: torch.Tensor, v_cache: torch.Tensor, kv_scales: Optional[tuple] = None) -> None:
         self.k_cache, self.v_cache, self.kv_scales = k_cache, v_cache, kv_scales
+
+    def read_by(self, window: int) -> None:
+        """Another layer reads this layer's cache through a window of ``window`` keys (0: all of them)."""
+        self.reach = max(self.reach, window) if self.reach and window else 0
 
     def kv_cache_shapes(self, num_blocks: int, block_size: int):
         """Shapes of this layer's two cache tensors."""
@@ -285,6 +292,8 @@ class RowLatentAttention(Attention):
         if source is not None and (source.rank, source.rope) != (rank, rope):
             raise ValueError(f"layer {layer_idx} reads the latent rows of layer {source.layer_idx}, which have "
                              f"another shape ({source.rank} + {source.rope} against {rank} + {rope})")
+        if source is not None:
+            source.read_by(self.window)
         # (kept out of the module tree: the owner is registered where it lives)
         object.__setattr__(self, "source", source)
 
@@ -339,18 +348,30 @@ class WindowBiasAttention(Attention):
     by blocks of ``chunk`` positions counted from the sequence's start: a query sees the keys of its own block up to
     itself (``window`` is then ``chunk``: no key further back is ever read, so the pages behind it are given back).
     ``sink`` may be another instance's parameter (layers that run several times over one set of weights), or a float: a
-    fixed score for every head (0.0: one is added to the denominator)."""
+    fixed score for every head (0.0: one is added to the denominator).  ``source``: another layer's instance whose keys
+    and values this layer reads, with queries, mask, scale and everything else of its own (the reader allocates nothing
+    and writes nothing)."""
     row_cache = True
 
     def __init__(self, num_heads: int, dim: int, vdim: int, num_kv_heads: int, scale: float, layer_idx: int,
                  window: int = 0, keep_first: int = 0, softcap: Optional[float] = None, distance_bias: bool = True,
-                 sink=True, chunk: int = 0):
+                 sink=True, chunk: int = 0, source: Optional["WindowBiasAttention"] = None):
         self.chunk = int(chunk or 0)
         if self.chunk:
             window, keep_first = self.chunk, 0
         super().__init__(num_heads, dim, num_kv_heads, scale, layer_idx, sliding_window=window, softcap=softcap)
         self.vdim = vdim
         self.keep_first = int(keep_first or 0) if self.window else 0
+        if source is not None:
+            if source.source is not None:
+                raise ValueError(f"layer {layer_idx} reads the keys of layer {source.layer_idx}, which has none of its own")
+            mine, theirs = (num_kv_heads, dim, vdim), (source.num_kv_heads, source.head_dim, source.vdim)
+            if mine != theirs:
+                raise ValueError(f"layer {layer_idx} reads the keys and values of layer {source.layer_idx}, which have "
+                                 f"another shape (heads, key size, value size: {theirs} against {mine})")
+            source.read_by(self.window)
+        # (kept out of the module tree: the owner is registered where it lives)
+        object.__setattr__(self, "source", source)
         f32 = torch.float32
         # (fp32 whatever the model dtype: they enter the scores directly)
         self.bias_scale = nn.Parameter(torch.zeros(num_heads, dtype=f32), requires_grad=False) if distance_bias else None
@@ -386,13 +407,14 @@ class WindowBiasAttention(Attention):
         out = torch.empty((t, self.num_heads, self.vdim), dtype=q.dtype, device=q.device)
         pos = _CTX.positions
         nd, nb = md.num_decode_tokens, md.num_decodes
+        own = self.source if self.source is not None else self
         common = (self.scale, self.softcap, self.window, self.keep_first, self.bias_scale, self.bias_rate, self.sink)
         if nd > 0:            # one row per sequence: the waves of a block share its keys
-            ops.window_bias_attention(q[:nd], self.k_cache, self.v_cache, md.block_table[:nb], md.query_start_loc[:nb + 1],
+            ops.window_bias_attention(q[:nd], own.k_cache, own.v_cache, md.block_table[:nb], md.query_start_loc[:nb + 1],
                                       md.seq_lens[:nb], None, pos[:nd], *common,
                                       None if gate is None else gate[:nd], 1, out=out[:nd], chunk=self.chunk)
         if md.num_prefills > 0:
-            ops.window_bias_attention(q[nd:], self.k_cache, self.v_cache, md.block_table[nb:],
+            ops.window_bias_attention(q[nd:], own.k_cache, own.v_cache, md.block_table[nb:],
                                       md.prefill_query_start_loc, md.seq_lens[nb:], md.prefill_token_rows(pos), pos[nd:],
                                       *common, None if gate is None else gate[nd:], md.max_prefill_query_len,
                                       out=out[nd:], chunk=self.chunk)
@@ -457,7 +479,8 @@ class ResidualRMSNorm(nn.Module):
     checkpoint keeps the gain minus one).  ``forward`` returns the model dtype (the input of a projection); ``add`` folds one or
     two sublayer outputs into the stream and hands back the normed sum in the same launch; ``after`` does so for an
     output that is itself RMS-normed with ``post_weight`` before it joins the stream, ``fold`` for an output that THIS
-    norm is for."""
+    norm is for, ``after_pair`` for two normed outputs (each with a weight of its own, their sum scaled) beside an
+    output that joins as it is."""
 
     def __init__(self, hidden_size: int, eps: float, dtype: torch.dtype, offset: float = 0.0):
         super().__init__()
@@ -472,6 +495,12 @@ class ResidualRMSNorm(nn.Module):
 
     def after(self, y: torch.Tensor, post_weight: torch.Tensor, residual: torch.Tensor) -> torch.Tensor:
         return ops.norm_add_norm(y, post_weight, residual, self.weight, self.eps, self.dtype, self.offset)
+
+    def after_pair(self, y: torch.Tensor, y_weight: torch.Tensor, z: torch.Tensor, z_weight: torch.Tensor, scale: float,
+                   plain: Optional[torch.Tensor], residual: torch.Tensor) -> torch.Tensor:
+        """``residual += scale * (norm(y) y_weight + norm(z) z_weight) + plain``; this norm of the sum.  One launch."""
+        return ops.norm_add_norm(y, y_weight, residual, self.weight, self.eps, self.dtype, self.offset, True, scale,
+                                 (z, z_weight), plain)
 
     def fold(self, y: torch.Tensor, residual: torch.Tensor, scale: float = 1.0,
              then: Optional["ResidualRMSNorm"] = None) -> torch.Tensor:

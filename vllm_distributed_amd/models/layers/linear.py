@@ -413,6 +413,40 @@ class QKVParallelLinear(_LinearBase):
         return self._matmul(x, self.bias)
 
 
+class GroupedColumnLinear(ColumnParallelLinear):
+    """Projections of several consumers of one input as ONE matrix: ``groups`` lists each consumer's sub-matrix sizes, and a
+    group that does not end on a multiple of 8 columns is followed by zero rows, so that every consumer's columns start (and
+    every row of the result does) on a 16-byte border in 16-bit types.  ``shard(group, i)`` is the loader's index of a
+    sub-matrix, ``columns(group)`` its group's column range (without the padding)."""
+
+    def __init__(self, in_features: int, groups: Sequence[Sequence[int]], dtype: torch.dtype):
+        sizes, self._first, self._cols, self._pads = [], [], [], []
+        for g in groups:
+            lo = sum(sizes)
+            self._first.append(len(sizes))
+            self._cols.append((lo, lo + sum(g)))
+            sizes += list(g)
+            pad = -sum(sizes) % 8
+            if pad:
+                self._pads.append(len(sizes))
+                sizes.append(pad)
+        super().__init__(in_features, sizes, False, dtype)
+        if self.tp > 1:
+            raise NotImplementedError("GroupedColumnLinear runs unsharded")
+
+    def shard(self, group: int, i: int) -> int:
+        return self._first[group] + i
+
+    def columns(self, group: int) -> Tuple[int, int]:
+        return self._cols[group]
+
+    def finalize_weights(self) -> None:
+        for p in self._pads:
+            lo = sum(self.shard_sizes[:p])
+            self.weight.data[lo:lo + self.shard_sizes[p]].zero_()
+        super().finalize_weights()
+
+
 class RowParallelLinear(_LinearBase):
     def __init__(self, in_features: int, out_features: int, bias: bool, dtype: torch.dtype,
                  reduce_results: bool = True):

@@ -1,4 +1,4 @@
-"""Linear attention with a recurrent state per request: a decay per head, the gated delta rule, a state-space
+"""Linear attention with a recurrent state per request: a decay per head or per key channel, the gated delta rule, a state-space
 recurrence whose decay depends on the token (per head, or per channel and state), or a gated linear unit per channel.
 
 Per head ``S_t = decay[h] * S_(t-1) + k_t v_t^T`` and ``o_t = S_t^T q_t``: no softmax, no cache that grows with the
@@ -53,6 +53,37 @@ class DecayLinearAttention(nn.Module):
         return ops.decay_linear_attention(x, self.num_heads, self.dim, self.vdim, self.decay, self.state,
                                           md.state_slots, md.query_start_loc, md.seq_lens, self.activation,
                                           md.max_query_len)
+
+
+class GatedLinearHeads(nn.Module):
+    """Gated linear attention between its input projection and its output projection: per head ``S <- diag(alpha) S + k v^T``
+    and ``o = dim^-0.5 S^T q`` with a decay per head and key channel that comes from the token through a narrow middle,
+    ``alpha = sigmoid(a2 a + bias)^(1 / tau)``; then each head's RMS norm (``norm[vdim]``, shared) times ``silu(gate)``.
+    ``sizes``: the sub-matrices ``[q | k | v | gate | a]`` whose products ``forward`` reads side by side (the caller may
+    fuse them with those of other consumers of the same input).  The state tensor is a ``layers.short_conv.SlotState``."""
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, rank: int, tau: float, eps: float, layer_idx: int,
+                 dtype: torch.dtype):
+        super().__init__()
+        self.heads, self.dim, self.vdim, self.rank, self.tau = heads, dim, vdim, rank, float(tau)
+        self.eps, self.dtype, self.layer_idx = eps, dtype, layer_idx
+        self.sizes, self.out_cols = [heads * dim, heads * dim, heads * vdim, heads * vdim, rank], heads * vdim
+        self.a2 = ReplicatedLinear(rank, heads * dim, False, dtype)
+        self.a2_bias = nn.Parameter(torch.zeros(heads * dim, dtype=torch.float32), requires_grad=False)
+        self.norm = nn.Parameter(torch.zeros(vdim, dtype=torch.float32), requires_grad=False)
+        self.slot_state = SlotState((heads, dim, vdim), torch.float32)
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        """``x[T, sum(sizes)]`` (rows may be strided) -> the gated heads ``[T, heads * vdim]``."""
+        md = get_forward_context().attn_metadata
+        vs = self.heads * self.vdim
+        if md is None:                    # memory-profiling pass: no state bound
+            return x.new_zeros((x.shape[0], vs))
+        lo = 2 * self.heads * self.dim + vs
+        alpha = ops.low_rank_decay(x[:, lo + vs:lo + vs + self.rank], self.a2.weight, self.a2_bias, self.tau)
+        o = ops.decay_linear_attention(x, self.heads, self.dim, self.vdim, alpha, self.slot_state.state, md.state_slots,
+                                       md.query_start_loc, md.seq_lens, False, md.max_query_len, self.dim ** -0.5)
+        return ops.gated_rms_norm(o, self.norm, x[:, lo:lo + vs], self.eps, self.dtype, group=self.vdim, silu=True)
 
 
 class GatedDeltaRule(nn.Module):

@@ -502,28 +502,37 @@ class GroupedIdentityMoE(FusedMoE):
                                    self.real_experts, shared, gate)
 
 
-class BiasedTopKMoE(FusedMoE):
-    """Routed experts of the plain form ``down(act(up(x)))`` (no gate projection, no biases) behind a router with a
-    bias: the ``top_k`` largest of ``router(x) + bias`` are chosen and weighted by the softmax over just those.
+class PlainTopKMoE(FusedMoE):
+    """Routed experts of the plain form ``down(act(up(x)))`` (no gate projection, no biases).  ``scores`` ``"softmax"``: the
+    ``top_k`` largest router outputs (plus a bias with ``router_bias``) are chosen and weighted by the softmax over just
+    those; ``"sigmoid"``: every output is scored by its sigmoid, the ``top_k`` largest scores are chosen and ARE the weights.
+    ``weigh_input``: a weight multiplies its expert's input (formed as the weighted output of the up projection, which has
+    no bias: the same number without rounding the weighted input) and the experts' outputs are summed as they are.
 
-    The router is fp32 (product and bias).  On the GPU in 16-bit types the experts run as two grouped GEMMs over
+    The router is fp32 (product, bias and scores).  On the GPU in 16-bit types the experts run as two grouped GEMMs over
     expert-sorted rows, their reduction dimensions zero-padded to the kernels' 128-deep tiles; elsewhere (fp32, CPU)
-    one after the other on the library GEMM.  ``activation``: ``"gelu"`` (exact) or ``"gelu_tanh"``."""
+    one after the other on the library GEMM.  ``activation``: ``"gelu"`` (exact), ``"gelu_tanh"`` or ``"relu2"`` (the
+    squared ReLU)."""
     custom_routing = True
 
     def __init__(self, hidden: int, inter: int, num_experts: int, top_k: int, dtype: torch.dtype,
-                 activation: str = "gelu"):
+                 activation: str = "gelu", scores: str = "softmax", router_bias: bool = False, weigh_input: bool = False):
         super().__init__(hidden, inter, num_experts, top_k, True, dtype, expert_parallel=False, allocate_experts=False)
         if self.tp > 1:
-            raise NotImplementedError("BiasedTopKMoE runs unsharded")
+            raise NotImplementedError(f"{type(self).__name__} runs unsharded")
         if not 1 <= top_k <= num_experts:
             raise ValueError(f"top {top_k} of {num_experts} experts")
-        if activation not in ("gelu", "gelu_tanh"):
+        if activation not in ("gelu", "gelu_tanh", "relu2"):
             raise ValueError(f"unsupported expert activation {activation!r}")
+        if scores not in ("softmax", "sigmoid"):
+            raise ValueError(f"unsupported router scores {scores!r}")
+        if weigh_input and activation != "relu2":
+            raise NotImplementedError("weights on the experts' inputs are written for the squared ReLU")
         self.quant = None
-        self.tanh = activation == "gelu_tanh"
+        self.act, self.sigmoid, self.weigh_input = activation, scores == "sigmoid", bool(weigh_input)
         self.gate = ReplicatedLinear(hidden, num_experts, False, dtype, quant=False)
-        self.gate_bias = nn.Parameter(torch.zeros(num_experts, dtype=torch.float32), requires_grad=False)
+        self.gate_bias = (nn.Parameter(torch.zeros(num_experts, dtype=torch.float32), requires_grad=False)
+                          if router_bias else None)
         self.h_pad, self.i_pad = _ceil128(hidden), _ceil128(inter)
         self.w1 = nn.Parameter(torch.zeros(num_experts, self.i_pad, self.h_pad, dtype=dtype), requires_grad=False)
         self.w2 = nn.Parameter(torch.zeros(num_experts, hidden, self.i_pad, dtype=dtype), requires_grad=False)
@@ -539,17 +548,27 @@ class BiasedTopKMoE(FusedMoE):
         param.data[int(shard_id), :, :self.inter].copy_(materialize(w))
 
     def router_logits(self, x: torch.Tensor) -> torch.Tensor:
-        return ops.linear_f32(x, self.gate.weight) + self.gate_bias
+        logits = ops.linear_f32(x, self.gate.weight)
+        return logits if self.gate_bias is None else logits + self.gate_bias
 
     def route(self, logits: torch.Tensor):
+        if self.sigmoid:
+            val, topi = torch.sigmoid(logits.float()).topk(self.top_k, dim=-1)
+            return val, topi
         val, topi = logits.float().topk(self.top_k, dim=-1)
         return torch.softmax(val, dim=-1), topi
 
     def _pad(self, x: torch.Tensor) -> torch.Tensor:
         return x if self.h_pad == self.hidden else F.pad(x, (0, self.h_pad - self.hidden))
 
-    def _expert_mlp(self, e: int, x: torch.Tensor) -> torch.Tensor:
-        return F.linear(ops.gelu(F.linear(self._pad(x), self.w1[e]), self.tanh), self.w2[e])
+    def _activate(self, h: torch.Tensor) -> torch.Tensor:
+        return ops.relu_squared(h) if self.act == "relu2" else ops.gelu(h, self.act == "gelu_tanh")
+
+    def _expert_mlp(self, e: int, x: torch.Tensor, weights: Optional[torch.Tensor] = None) -> torch.Tensor:
+        h = F.linear(self._pad(x), self.w1[e])
+        if weights is not None:
+            h = (h.float() * weights.unsqueeze(1)).to(h.dtype)
+        return F.linear(self._activate(h), self.w2[e])
 
     def _grouped_tile_rows(self, x: torch.Tensor) -> int:
         if not (x.is_cuda and x.dtype in (torch.bfloat16, torch.float16) and x.dim() == 2 and ops.hip_available()):
@@ -573,13 +592,16 @@ class BiasedTopKMoE(FusedMoE):
         logits = self.router_logits(x)
         tile_rows = self._grouped_tile_rows(x)
         if tile_rows:
-            # (softmax over every output, the largest kept and renormalised: the softmax over the kept ones)
-            topw, topi = ops.moe_topk(logits, self.top_k, True)
+            if self.sigmoid:
+                topw, topi = ops.moe_topk_grouped(logits, None, self.top_k, 1, 1, True, False, False, 1.0)
+            else:                        # (softmax over every output, the largest kept and renormalised: the softmax over them)
+                topw, topi = ops.moe_topk(logits, self.top_k, True)
             src_row, inv, tiles = ops.moe_align_fused(topi, self.num_experts, tile_rows, 0, -1)
             xs = self._pad(x).index_select(0, src_row)
             h = ops.grouped_linear(xs, tiles, tile_rows, weight=self.w1)
-            y = ops.grouped_linear(ops.gelu(h, self.tanh), tiles, tile_rows, weight=self.w2)
-            return ops.moe_combine(y, topw, topi, inv, 0, -1)
+            h = ops.weighted_relu_squared(h, topw, inv) if self.weigh_input else self._activate(h)
+            y = ops.grouped_linear(h, tiles, tile_rows, weight=self.w2)
+            return ops.moe_combine(y, None if self.weigh_input else topw, topi, inv, 0, -1)
         topw, topi = self.route(logits)
         acc = torch.zeros(x.shape, dtype=torch.float32, device=x.device)
         flat_e = topi.reshape(-1)
@@ -592,9 +614,22 @@ class BiasedTopKMoE(FusedMoE):
             if n:
                 seg = slice(start, start + n)
                 rows = tok[seg]
-                acc.index_add_(0, rows, self._expert_mlp(eid, x.index_select(0, rows)).float() * wts[seg].unsqueeze(1))
+                xe = x.index_select(0, rows)
+                if self.weigh_input:
+                    acc.index_add_(0, rows, self._expert_mlp(eid, xe, wts[seg]).float())
+                else:
+                    acc.index_add_(0, rows, self._expert_mlp(eid, xe).float() * wts[seg].unsqueeze(1))
             start += n
         return acc.to(x.dtype)
+
+
+class BiasedTopKMoE(PlainTopKMoE):
+    """Plain experts with a GELU behind a router with a bias: the softmax over the ``top_k`` largest of ``router(x) + bias``
+    weighs their outputs."""
+
+    def __init__(self, hidden: int, inter: int, num_experts: int, top_k: int, dtype: torch.dtype,
+                 activation: str = "gelu"):
+        super().__init__(hidden, inter, num_experts, top_k, dtype, activation, router_bias=True)
 
 
 class GatedMLP(nn.Module):

@@ -1,10 +1,11 @@
-"""Two sequence mixers side by side on one input, their output projections fused into one."""
+"""Two sequence mixers side by side on one input: their output projections fused into one, or their input projections fused
+and their outputs kept apart (each is normed before they meet)."""
 from __future__ import annotations
 
 import torch
 import torch.nn as nn
 
-from .linear import RowParallelLinear
+from .linear import GroupedColumnLinear, RowParallelLinear
 
 
 class ParallelHeads(nn.Module):
@@ -29,3 +30,25 @@ class ParallelHeads(nn.Module):
         self.left(h, index, heads[:, :nl])
         self.right(h, index, heads[:, nl:])
         return self.o(heads)
+
+
+class ParallelNormed(nn.Module):
+    """``left`` and ``right`` read the same input through ONE projection; their outputs, each ``o(heads)`` in the model
+    width, are RMS-normed on their own (gains ``left_out`` / ``right_out``) before they join the residual stream, which the
+    caller does in the launch that also adds the feed-forward (``layers.attention.ResidualRMSNorm.after_pair``).  Each
+    half has ``sizes`` (its sub-matrices of the projection), ``out_cols`` and ``forward(columns) -> heads``."""
+
+    def __init__(self, left: nn.Module, right: nn.Module, width: int, dtype: torch.dtype):
+        super().__init__()
+        self.left, self.right = left, right
+        self.proj = GroupedColumnLinear(width, [left.sizes, right.sizes], dtype)
+        self.left_o = RowParallelLinear(left.out_cols, width, False, dtype)
+        self.right_o = RowParallelLinear(right.out_cols, width, False, dtype)
+        f32 = torch.float32
+        self.left_out = nn.Parameter(torch.zeros(width, dtype=f32), requires_grad=False)
+        self.right_out = nn.Parameter(torch.zeros(width, dtype=f32), requires_grad=False)
+
+    def forward(self, h: torch.Tensor):
+        x = self.proj(h)
+        (l0, l1), (r0, r1) = self.proj.columns(0), self.proj.columns(1)
+        return self.left_o(self.left(x[:, l0:l1])), self.right_o(self.right(x[:, r0:r1]))

@@ -63,6 +63,9 @@ def _weight_shapes(c: dict, arch: str) -> Dict[str, Tuple[int, ...]]:
     if arch in ("KefuraxForCausalLM", "Kefurax"):
         from .kefurax import weight_shapes
         return weight_shapes(c)
+    if arch in ("BapovikForCausalLM", "Bapovik"):
+        from .bapovik import weight_shapes
+        return weight_shapes(c)
     if arch == "MedusaModel":
         h = c["hidden_size"]
         out = {}
@@ -482,6 +485,10 @@ def dummy_weights_iterator(mc: ModelConfig, device: torch.device,
             continue
         if mc.architecture in ("KefuraxForCausalLM", "Kefurax"):
             from .kefurax import random_weight
+            yield name, random_weight(name, shape, gen, device, dtype)
+            continue
+        if mc.architecture in ("BapovikForCausalLM", "Bapovik"):
+            from .bapovik import random_weight
             yield name, random_weight(name, shape, gen, device, dtype)
             continue
         if awq and _QUANTIZED_LINEAR.search(name) and shape[1] % g == 0 and shape[0] % 8 == 0:

@@ -84,6 +84,11 @@ _MODELS: Dict[str, Tuple[str, str]] = {
     # scan per channel, attention over rotated-then-normed heads beside the gated delta rule
     "KefuraxForCausalLM": ("kefurax", "KefuraxForCausalLM"),
     "Kefurax": ("kefurax", "KefuraxForCausalLM"),
+    # fp32 residual stream; mixer and experts side by side on one normed input; chunked attention with capped scores beside
+    # gated linear attention (each half's output normed), windowed attention whose keys another layer may read; experts
+    # that weigh their input
+    "BapovikForCausalLM": ("bapovik", "BapovikForCausalLM"),
+    "Bapovik": ("bapovik", "BapovikForCausalLM"),
     # draft heads of speculative decoding (never a served model by themselves; worker/draft_model.py)
     "EagleLlamaForCausalLM": ("spec_heads", "EagleLlamaForCausalLM"),
     "Eagle3LlamaForCausalLM": ("spec_heads", "Eagle3LlamaForCausalLM"),
@@ -96,7 +101,8 @@ _MODELS: Dict[str, Tuple[str, str]] = {
 # architectures whose layers keep per-request state besides the KV cache (convolution tails, recurrences): a cached
 # prefix's blocks do not bring that state back, so prefix reuse is off for them
 _KEEPS_REQUEST_STATE = {"TavulixForCausalLM", "Tavulix", "KabapelForCausalLM", "Kabapel", "GosizenForCausalLM",
-                        "Gosizen", "NalasunForCausalLM", "Nalasun", "KefuraxForCausalLM", "Kefurax"}
+                        "Gosizen", "NalasunForCausalLM", "Nalasun", "KefuraxForCausalLM", "Kefurax",
+                        "BapovikForCausalLM", "Bapovik"}
 
 
 def keeps_request_state(arch: str) -> bool:

@@ -714,13 +714,28 @@ def add_layer_norm(y, residual, weight, bias, eps: float, out_dtype):
 
 
 def decay_linear_attention(x, num_heads: int, dim: int, vdim: int, decay, state, slots, query_start_loc, seq_lens,
-                           silu: bool = True, max_query_len: int = 0):
-    """Linear attention with a per-head decay and a per-request fp32 state; see
-    ``torch_ref.decay_linear_attention``.  ``max_query_len`` (0: unknown) only helps the kernel choose its launch."""
+                           silu: bool = True, max_query_len: int = 0, scale: float = 1.0):
+    """Linear attention with a decay per head, or per row, head and key channel (``decay`` 2-D), and a per-request fp32
+    state; see ``torch_ref.decay_linear_attention``.  ``max_query_len`` (0: unknown) only helps the kernel choose its launch."""
     if _use_hip(x):
         return _hip.decay_linear_attention(x, num_heads, dim, vdim, decay, state, slots, query_start_loc, seq_lens,
-                                           silu, max_query_len)
-    return torch_ref.decay_linear_attention(x, num_heads, dim, vdim, decay, state, slots, query_start_loc, seq_lens, silu)
+                                           silu, max_query_len, scale)
+    return torch_ref.decay_linear_attention(x, num_heads, dim, vdim, decay, state, slots, query_start_loc, seq_lens, silu,
+                                            scale)
+
+
+def low_rank_decay(a, weight, bias, tau: float):
+    """``sigmoid(a @ weight^T + bias)^(1 / tau)`` in fp32, fp32 result; see ``torch_ref.low_rank_decay``."""
+    if _use_hip(a):
+        return _hip.low_rank_decay(a, weight, bias, tau)
+    return torch_ref.low_rank_decay(a, weight, bias, tau)
+
+
+def weighted_relu_squared(h, topw, inv):
+    """``max(w h, 0)^2`` of expert-sorted rows with each row's routing weight; see ``torch_ref.weighted_relu_squared``."""
+    if _use_hip(h):
+        return _hip.weighted_relu_squared(h, topw, inv)
+    return torch_ref.weighted_relu_squared(h, topw, inv)
 
 
 def gated_rms_norm(o, weight, gate, eps: float, out_dtype, group: int = 0, scale: float = 1.0, out=None,
@@ -790,14 +805,15 @@ def add_rms_norm_to(residual, a, b, weight, eps: float, out_dtype, offset: float
 
 
 def norm_add_norm(y, post_weight, residual, next_weight, eps: float, out_dtype, next_offset: float = 0.0,
-                  next_normed: bool = True, post_scale: float = 1.0):
+                  next_normed: bool = True, post_scale: float = 1.0, second=None, plain=None):
     """``residual += post_scale * rms_norm(y) * post_weight`` on the fp32 residual stream and the RMS norm of the sum
-    (or the sum itself) in ``out_dtype``: one launch."""
+    (or the sum itself) in ``out_dtype``: one launch.  ``second`` = ``(z, weight)`` joins the same way, ``plain`` as it
+    is."""
     if _use_hip(y):
         return _hip.norm_add_norm(y, post_weight, residual, next_weight, eps, out_dtype, next_offset, next_normed,
-                                  post_scale)
+                                  post_scale, second, plain)
     return torch_ref.norm_add_norm(y, post_weight, residual, next_weight, eps, out_dtype, next_offset, next_normed,
-                                   post_scale)
+                                   post_scale, second, plain)
 
 
 def gelu_mul_rows(g, table, ids, col: int):
@@ -904,13 +920,15 @@ def mix_heads(o, talk, out_dtype):
 # ------------------------------------------------ rotation in front of a head norm, a selective scan per channel, a
 # ------------------------------------------------ gated linear unit recurrence
 def rotate_norm_cache(x, num_heads: int, num_kv_heads: int, dim: int, vdim: int, inv_freq, rot_scale: float,
-                      interleaved: bool, eps: float, q_norm, k_norm, positions, k_cache, v_cache, slot_mapping):
-    """q and k heads rotated, then normed, k and v into the row caches; see ``torch_ref.rotate_norm_cache``."""
+                      interleaved: bool, eps: float, q_norm, k_norm, positions, k_cache, v_cache, slot_mapping,
+                      normed: bool = True, bias=None):
+    """q and k heads biased, rotated, then normed (each optional), k and v into the row caches; see
+    ``torch_ref.rotate_norm_cache``."""
     if _use_hip(x):
         return _hip.rotate_norm_cache(x, num_heads, num_kv_heads, dim, vdim, inv_freq, rot_scale, interleaved, eps,
-                                      q_norm, k_norm, positions, k_cache, v_cache, slot_mapping)
+                                      q_norm, k_norm, positions, k_cache, v_cache, slot_mapping, normed, bias)
     return torch_ref.rotate_norm_cache(x, num_heads, num_kv_heads, dim, vdim, inv_freq, rot_scale, interleaved, eps,
-                                       q_norm, k_norm, positions, k_cache, v_cache, slot_mapping)
+                                       q_norm, k_norm, positions, k_cache, v_cache, slot_mapping, normed, bias)
 
 
 def gelu_and_mul(x, tanh: bool = True):

@@ -70,13 +70,13 @@ def load() -> ctypes.CDLL:
         "vdamd_poly_norm": [P, P, P, F, I, I, L, I, P],
         "vdamd_conv_norm_cache": [P, L] + [P] * 16 + [I] * 8 + [F, I, P, I, I, P],
         "vdamd_short_conv_act": [P, L, P, L, P, P, P, P, P, P, P] + [I] * 6 + [P, I, P, I, P],
-        "vdamd_rotate_norm_cache": [P, P, L, P, I, F, I, F] + [P] * 6 + [I] * 7 + [P],
+        "vdamd_rotate_norm_cache": [P, P, L, P, I, F, I, F] + [P] * 7 + [I] * 8 + [P],
         "vdamd_window_bias_attention": [P, P, P, P, L, P, P, P, P, P, P, P, P, L, P] + [I] * 10 + [F, F, I, I, I, I, P],
         "vdamd_selective_scan": [P, P, L, P, L, P, P, P, P, P, P, P] + [I] * 7 + [P],
         "vdamd_act_gate_group_norm": [P, P, P, L, P, F, I, I, I, I, P],
         "vdamd_joint_norm_cache": [P, P, L, P, P, F, P, F, I, P, P, P] + [I] * 6 + [P],
         "vdamd_mix_heads": [P, P, P, I, I, I, I, I, P],
-        "vdamd_residual_rms": [P, L, P, L, P, L, P, L, P, L, P, P, F, F, I, I, I, I, I, I, F, P],
+        "vdamd_residual_rms": [P, L, P, L, P, L, P, L, P, L, P, L, P, P, P, F, F, I, I, I, I, I, I, F, P],
         "vdamd_gelu_and_mul": [P, P, L, I, I, I, I, P],
         "vdamd_channel_scan": [P, P, L, P, L, P, L, P, L] + [P] * 7 + [I] * 6 + [P],
         "vdamd_block_gates_mfma_ok": [I, I],
@@ -94,6 +94,9 @@ def load() -> ctypes.CDLL:
         "vdamd_relu_squared": [P, P, L, I, P],
         "vdamd_expert_epilogue": [P, P, P, L, P, P, I, I, P, P, L, I, I, I, P],
         "vdamd_decay_linear_attention": [P, P, L, P, P, P, P, P, I, I, I, I, I, I, I, P],
+        "vdamd_channel_decay_attention": [P, P, L, P, P, P, P, P, I, I, I, I, F, I, I, I, P],
+        "vdamd_low_rank_decay": [P, P, L, P, P, I, I, I, F, I, P],
+        "vdamd_weighted_relu_squared": [P, P, L, P, P, I, I, I, P],
         "vdamd_latent_prep": [P, P, L, L, I, P, L, L, P, L, P, F, P, I, F, P, P, P, P, I, I, I, I, I, I, I, P],
         "vdamd_latent_row_attention": [P, P, P, P, L, P, P, F, I, I, I, I, I, I, P, P, L, I, P],
     }
@@ -1057,9 +1060,9 @@ def moe_route_small(logits: torch.Tensor, x: torch.Tensor, k: int, renormalize: 
     return topw, topi, inv, tiles, xs
 
 
-def moe_combine(y: torch.Tensor, topw: torch.Tensor, topi: torch.Tensor, inv: torch.Tensor, expert_start: int = 0,
+def moe_combine(y: torch.Tensor, topw: Optional[torch.Tensor], topi: torch.Tensor, inv: torch.Tensor, expert_start: int = 0,
                 local_experts: int = -1, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``out[t] = sum_j topw[t, j] * y[inv[t*k + j]]`` in fp32 (slots of experts this rank does not hold are skipped).
+    """``out[t] = sum_j topw[t, j] * y[inv[t*k + j]]`` in fp32 (``topw`` None: weights of one; slots of experts this rank does not hold are skipped).
     ``bias [local experts, H]``: each row first gains its expert's bias (rounded to the row's dtype)."""
     t, k = topi.shape
     h = y.shape[1]
@@ -1067,9 +1070,10 @@ def moe_combine(y: torch.Tensor, topw: torch.Tensor, topi: torch.Tensor, inv: to
         assert bias.dtype == y.dtype and bias.dim() == 2 and bias.shape[1] == h and bias.is_contiguous()
         assert bias.shape[0] >= (local_experts if local_experts >= 0 else 1)
     assert _half(y) and y.stride(1) == 1 and y.stride(0) % 8 == 0 and h % 8 == 0 and y.data_ptr() % 16 == 0
-    assert topw.dtype == torch.float32 and topw.is_contiguous() and topi.is_contiguous() and inv.numel() == t * k
+    assert topw is None or (topw.dtype == torch.float32 and topw.is_contiguous())
+    assert topi.is_contiguous() and inv.numel() == t * k
     out = torch.empty((t, h), dtype=y.dtype, device=y.device)
-    _check(_LIB.vdamd_moe_combine(out.data_ptr(), h, y.data_ptr(), y.stride(0), topw.data_ptr(), topi.data_ptr(),
+    _check(_LIB.vdamd_moe_combine(out.data_ptr(), h, y.data_ptr(), y.stride(0), _ptr(topw), topi.data_ptr(),
                                   inv.data_ptr(), t, k, h, expert_start, local_experts,
                                   None if bias is None else bias.data_ptr(), _dt(y), _stream()),
            "moe_combine")
@@ -1440,7 +1444,8 @@ DECAY_ATTENTION_MAX_DIM = 256
 
 def decay_linear_attention(x: torch.Tensor, num_heads: int, dim: int, vdim: int, decay: torch.Tensor,
                            state: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor,
-                           seq_lens: torch.Tensor, silu: bool = True, max_query_len: int = 0) -> torch.Tensor:
+                           seq_lens: torch.Tensor, silu: bool = True, max_query_len: int = 0,
+                           scale: float = 1.0) -> torch.Tensor:
     t = x.shape[0]
     n = seq_lens.numel()
     if dim > DECAY_ATTENTION_MAX_DIM:
@@ -1450,6 +1455,15 @@ def decay_linear_attention(x: torch.Tensor, num_heads: int, dim: int, vdim: int,
     assert slots.dtype == seq_lens.dtype == query_start_loc.dtype == torch.int32
     assert slots.numel() >= n and query_start_loc.numel() >= n + 1
     out = torch.empty((t, num_heads * vdim), dtype=torch.float32, device=x.device)
+    if decay.dim() == 2:                 # one per row, head and key channel
+        assert decay.shape == (t, num_heads * dim) and decay.dtype == torch.float32 and decay.is_contiguous()
+        _check(_LIB.vdamd_channel_decay_attention(
+            out.data_ptr(), x.data_ptr(), x.stride(0), decay.data_ptr(), state.data_ptr(), slots.data_ptr(),
+            query_start_loc.data_ptr(), seq_lens.data_ptr(), n, num_heads, dim, vdim, float(scale), int(bool(silu)),
+            int(max_query_len), _dt(x), _stream()), "channel_decay_attention")
+        return out
+    if scale != 1.0:
+        raise NotImplementedError("a scale on the result needs decays per key channel")
     _check(_LIB.vdamd_decay_linear_attention(out.data_ptr(), x.data_ptr(), x.stride(0),
                                              _f32_vec(decay, num_heads, "decay").data_ptr(), state.data_ptr(),
                                              slots.data_ptr(), query_start_loc.data_ptr(), seq_lens.data_ptr(), n,
@@ -1492,6 +1506,28 @@ def relu_squared(x: torch.Tensor) -> torch.Tensor:
     xc = x if x.is_contiguous() else x.contiguous()
     out = torch.empty_like(xc)
     _check(_LIB.vdamd_relu_squared(out.data_ptr(), xc.data_ptr(), xc.numel(), _dt(xc), _stream()), "relu_squared")
+    return out
+
+
+def low_rank_decay(a: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], tau: float) -> torch.Tensor:
+    rows, rank = _rows2d(a, "a").shape
+    c = weight.shape[0]
+    assert weight.shape == (c, rank) and weight.dtype == a.dtype and weight.is_contiguous()
+    out = torch.empty((rows, c), dtype=torch.float32, device=a.device)
+    _check(_LIB.vdamd_low_rank_decay(out.data_ptr(), a.data_ptr(), a.stride(0), weight.data_ptr(),
+                                     _ptr(_f32_vec(bias, c, "bias")), rows, c, rank, 1.0 / float(tau), _dt(a), _stream()),
+           "low_rank_decay")
+    return out
+
+
+def weighted_relu_squared(h: torch.Tensor, topw: torch.Tensor, inv: torch.Tensor) -> torch.Tensor:
+    rows, f = _rows2d(h, "h").shape
+    slots = topw.numel()
+    assert topw.dtype == torch.float32 and topw.is_contiguous() and rows >= slots
+    assert inv.dtype == torch.int32 and inv.is_contiguous() and inv.numel() == slots
+    out = torch.empty((rows, f), dtype=h.dtype, device=h.device)
+    _check(_LIB.vdamd_weighted_relu_squared(out.data_ptr(), h.data_ptr(), h.stride(0), topw.data_ptr(), inv.data_ptr(), slots,
+                                            f, _dt(h), _stream()), "weighted_relu_squared")
     return out
 
 
@@ -1582,24 +1618,27 @@ def _rows2d(t: torch.Tensor, name: str) -> torch.Tensor:
     return t
 
 
-def _residual_rms(x, a, b, y, post_w, w, eps, out_dtype, offset, normed, post_scale: float = 1.0) -> torch.Tensor:
+def _residual_rms(x, a, b, y, post_w, w, eps, out_dtype, offset, normed, post_scale: float = 1.0, z=None,
+                  post_w2=None) -> torch.Tensor:
     rows, h = _rows2d(x, "x").shape
     adds = a is not None or y is not None
     if adds:
         assert x.dtype == torch.float32, "the residual stream is fp32"
     in_dt = _dt(x)
-    for t, name in ((a, "a"), (b, "b"), (y, "y")):
+    for t, name in ((a, "a"), (b, "b"), (y, "y"), (z, "z")):
         if t is not None:
             assert _rows2d(t, name).shape == (rows, h)
             in_dt = _dt(t)
-    for u, v in ((a, b), (a, y), (b, y)):
+    for u, v in ((a, b), (a, y), (b, y), (y, z)):
         assert u is None or v is None or u.dtype == v.dtype
     assert b is None or a is not None
+    assert z is None or y is not None
     out = torch.empty((rows, h), dtype=out_dtype, device=x.device)
     _check(_LIB.vdamd_residual_rms(
         out.data_ptr(), h, x.data_ptr(), x.stride(0), _ptr(a), 0 if a is None else a.stride(0), _ptr(b),
-        0 if b is None else b.stride(0), _ptr(y), 0 if y is None else y.stride(0),
-        _ptr(_f32_vec(post_w, h, "post_weight")) if y is not None else None, _ptr(_f32_vec(w, h, "weight")),
+        0 if b is None else b.stride(0), _ptr(y), 0 if y is None else y.stride(0), _ptr(z), 0 if z is None else z.stride(0),
+        _ptr(_f32_vec(post_w, h, "post_weight")) if y is not None else None,
+        _ptr(_f32_vec(post_w2, h, "post_weight2")) if z is not None else None, _ptr(_f32_vec(w, h, "weight")),
         float(offset), float(eps), rows, h, 1 if normed else 0, _dt(x), in_dt, _DT[out_dtype],
         float(post_scale), _stream()), "residual_rms")
     return out
@@ -1618,10 +1657,11 @@ def add_rms_norm_to(residual, a, b, weight, eps: float, out_dtype, offset: float
 
 
 def norm_add_norm(y, post_weight, residual, next_weight, eps: float, out_dtype, next_offset: float = 0.0,
-                  next_normed: bool = True, post_scale: float = 1.0):
+                  next_normed: bool = True, post_scale: float = 1.0, second=None, plain=None):
     assert residual.is_contiguous()
-    return _residual_rms(residual, None, None, y, post_weight, next_weight, eps, out_dtype, next_offset, next_normed,
-                         post_scale)
+    z, w2 = second if second is not None else (None, None)
+    return _residual_rms(residual, plain, None, y, post_weight, next_weight, eps, out_dtype, next_offset, next_normed,
+                         post_scale, z, w2)
 
 
 def gelu_mul_rows(g: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, col: int) -> torch.Tensor:
@@ -1783,10 +1823,11 @@ def mix_heads(o: torch.Tensor, talk: torch.Tensor, out_dtype: torch.dtype) -> to
 # ------------------------------------------------ gated linear unit recurrence
 def rotate_norm_cache(x, num_heads: int, num_kv_heads: int, dim: int, vdim: int, inv_freq, rot_scale: float,
                       interleaved: bool, eps: float, q_norm, k_norm, positions, k_cache, v_cache,
-                      slot_mapping) -> torch.Tensor:
+                      slot_mapping, normed: bool = True, bias=None) -> torch.Tensor:
     t = _rows2d(x, "x").shape[0]
     h, g, d, dv = int(num_heads), int(num_kv_heads), int(dim), int(vdim)
-    assert x.shape[1] >= (h + g) * d + g * dv and positions.shape[0] >= t and h % g == 0 and d <= UNIT_MAX_WIDTH
+    assert x.shape[1] >= (h + g) * d + g * dv and positions.shape[0] >= t and d <= UNIT_MAX_WIDTH
+    assert (h % g == 0) if g else k_cache is None
     half = 0 if inv_freq is None else int(inv_freq.numel())
     assert 2 * half <= d
     bs = 0
@@ -1800,9 +1841,10 @@ def rotate_norm_cache(x, num_heads: int, num_kv_heads: int, dim: int, vdim: int,
     _check(_LIB.vdamd_rotate_norm_cache(
         q.data_ptr(), x.data_ptr(), x.stride(0), _ptr(_f32_vec(inv_freq, half, "inv_freq")) if half else None, half,
         float(rot_scale), 1 if interleaved else 0, float(eps), _ptr(_f32_vec(q_norm, d, "q_norm")),
-        _ptr(_f32_vec(k_norm, d, "k_norm")), _i32(positions, "positions").data_ptr(), _ptr(k_cache), _ptr(v_cache),
-        _ptr(_i32(slot_mapping, "slot_mapping") if k_cache is not None else None), t, h, g, d, dv, int(bs), _dt(x),
-        _stream()), "rotate_norm_cache")
+        _ptr(_f32_vec(k_norm, d, "k_norm")), _ptr(_f32_vec(bias, (h + g) * d + g * dv, "bias")),
+        _i32(positions, "positions").data_ptr(), _ptr(k_cache), _ptr(v_cache),
+        _ptr(_i32(slot_mapping, "slot_mapping") if k_cache is not None else None), t, h, g, d, dv, int(bs),
+        1 if normed else 0, _dt(x), _stream()), "rotate_norm_cache")
     return q
 
 

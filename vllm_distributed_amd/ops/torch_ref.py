@@ -628,10 +628,11 @@ def add_layer_norm(y: torch.Tensor, residual: torch.Tensor, weight: torch.Tensor
 
 def decay_linear_attention(x: torch.Tensor, num_heads: int, dim: int, vdim: int, decay: torch.Tensor,
                            state: torch.Tensor, slots: torch.Tensor, query_start_loc: torch.Tensor,
-                           seq_lens: torch.Tensor, silu: bool = True) -> torch.Tensor:
-    """Linear attention with one decay per head over the packed rows ``x[T, C]`` whose leading columns are
+                           seq_lens: torch.Tensor, silu: bool = True, scale: float = 1.0) -> torch.Tensor:
+    """Linear attention with one decay per head (``decay[H]``), or one per row, head and key channel (``decay[T, H *
+    dim]``, acting on the rows of the state), over the packed rows ``x[T, C]`` whose leading columns are
     ``[q (H * dim) | k (H * dim) | v (H * vdim)]`` (``silu``: each passed through SiLU first).  Per head
-    ``S_t = decay[h] S_(t-1) + k_t v_t^T`` and ``o_t = S_t^T q_t``; ``S`` is ``state[slots[i]]`` (``[slots, H, dim,
+    ``S_t = decay[h] S_(t-1) + k_t v_t^T`` and ``o_t = scale * S_t^T q_t``; ``S`` is ``state[slots[i]]`` (``[slots, H, dim,
     vdim]`` fp32) for sequence ``i``, taken as zero when the rows start at position 0 whatever the slot held, and left
     holding the state after the sequence's last row.  fp32 arithmetic; returns fp32 ``[T, H * vdim]``."""
     t = x.shape[0]
@@ -644,7 +645,7 @@ def decay_linear_attention(x: torch.Tensor, num_heads: int, dim: int, vdim: int,
     k = xf[:, qs:2 * qs].reshape(t, h, dim)
     v = xf[:, 2 * qs:].reshape(t, h, vdim)
     out = torch.zeros((t, h, vdim), dtype=torch.float32, device=x.device)
-    d = decay.float().view(h, 1, 1)
+    d = decay.float().view(h, 1, 1) if decay.dim() == 1 else decay.float().view(t, h, dim, 1)
     qsl, sls, sl = query_start_loc.tolist(), seq_lens.tolist(), slots.tolist()
     for i, n_ctx in enumerate(sls):
         s, e = qsl[i], qsl[i + 1]
@@ -652,10 +653,28 @@ def decay_linear_attention(x: torch.Tensor, num_heads: int, dim: int, vdim: int,
             continue
         st = state[sl[i]].float().clone() if n_ctx - (e - s) > 0 else torch.zeros_like(state[sl[i]], dtype=torch.float32)
         for r in range(s, e):
-            st = d * st + k[r].unsqueeze(2) * v[r].unsqueeze(1)
+            st = (d if decay.dim() == 1 else d[r]) * st + k[r].unsqueeze(2) * v[r].unsqueeze(1)
             out[r] = torch.einsum("hkv,hk->hv", st, q[r])
         state[sl[i]] = st.to(state.dtype)
-    return out.reshape(t, vs)
+    return out.reshape(t, vs) * scale
+
+
+def low_rank_decay(a: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], tau: float) -> torch.Tensor:
+    """Decays of channels from a narrow projection: ``sigmoid(a[T, r] @ weight[C, r]^T + bias)^(1 / tau)`` in fp32
+    arithmetic, fp32 ``[T, C]``."""
+    z = F.linear(a.float(), weight.float())
+    if bias is not None:
+        z = z + bias.float()
+    return torch.exp(F.logsigmoid(z) / tau)
+
+
+def weighted_relu_squared(h: torch.Tensor, topw: torch.Tensor, inv: torch.Tensor) -> torch.Tensor:
+    """``max(w h, 0)^2`` row by row for expert-sorted rows ``h[rows, F]``; ``inv[slot]`` is the row of (token, choice) slot
+    ``slot`` and ``topw[slot]`` its weight (rows of no slot: zero).  fp32 arithmetic, in ``h``'s dtype."""
+    out = torch.zeros_like(h)
+    rows = inv.reshape(-1).long()
+    out[rows] = torch.relu(h[rows].float() * topw.reshape(-1, 1).float()).square().to(h.dtype)
+    return out
 
 
 def gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, eps: float,
@@ -821,10 +840,16 @@ def add_rms_norm_to(residual: torch.Tensor, a: Optional[torch.Tensor], b: Option
 
 def norm_add_norm(y: torch.Tensor, post_weight: torch.Tensor, residual: torch.Tensor,
                   next_weight: Optional[torch.Tensor], eps: float, out_dtype: torch.dtype, next_offset: float = 0.0,
-                  next_normed: bool = True, post_scale: float = 1.0) -> Optional[torch.Tensor]:
+                  next_normed: bool = True, post_scale: float = 1.0, second=None,
+                  plain: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """``residual += post_scale * rms_norm(y) * post_weight`` in place on the fp32 residual stream; then what
-    ``add_rms_norm_to(residual, None, None, next_weight, ...)`` returns."""
+    ``add_rms_norm_to(residual, None, None, next_weight, ...)`` returns.  ``second`` = ``(z, weight)``: another output
+    that joins the same way; ``plain``: an output that joins as it is."""
     residual.add_(rms_norm_to(y, post_weight, eps, torch.float32), alpha=post_scale)
+    if second is not None:
+        residual.add_(rms_norm_to(second[0], second[1], eps, torch.float32), alpha=post_scale)
+    if plain is not None:
+        residual.add_(plain.float())
     if not next_normed:
         return residual.to(out_dtype)
     return rms_norm_to(residual, next_weight, eps, out_dtype, next_offset)
@@ -1028,21 +1053,29 @@ def rotate_norm_cache(x: torch.Tensor, num_heads: int, num_kv_heads: int, dim: i
                       inv_freq: Optional[torch.Tensor], rot_scale: float, interleaved: bool, eps: float,
                       q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], positions: torch.Tensor,
                       k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor],
-                      slot_mapping: Optional[torch.Tensor]) -> torch.Tensor:
+                      slot_mapping: Optional[torch.Tensor], normed: bool = True,
+                      bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """What lies between the fused projection ``x[T, >= C]`` = ``[q (H * dim) | k (Hkv * dim) | v (Hkv * vdim)]`` and the
     attention of a layer that rotates its heads BEFORE it norms them: the first ``2 * len(inv_freq)`` values of every
     q and k head turned by ``positions[t] * inv_freq[i]`` (cos and sin times ``rot_scale``; ``interleaved`` pairs
     neighbours), then the RMS norm of each head (``eps``; ``q_norm`` / ``k_norm`` ``[dim]`` gains or None: none), k and
-    v into ``k_cache[blocks, Hkv, block, dim]`` and ``v_cache[blocks, Hkv, block / 8, vdim, 8]``.  fp32 arithmetic;
-    returns ``q[T, H, dim]`` in ``x``'s dtype."""
+    v into ``k_cache[blocks, Hkv, block, dim]`` and ``v_cache[blocks, Hkv, block / 8, vdim, 8]``.  ``bias[C]`` joins the
+    projection first; ``normed`` False: no head norm; ``num_kv_heads`` 0: queries only, nothing is cached.  fp32
+    arithmetic; returns ``q[T, H, dim]`` in ``x``'s dtype."""
     t = x.shape[0]
     qs, ks = num_heads * dim, num_kv_heads * dim
+    if bias is not None:
+        c = qs + ks + num_kv_heads * vdim
+        dtype, x = x.dtype, x[:, :c].float() + bias.float()
+    else:
+        dtype = x.dtype
     q = x[:, :qs].float().reshape(t, num_heads, dim)
     k = x[:, qs:qs + ks].float().reshape(t, num_kv_heads, dim)
     if inv_freq is not None and inv_freq.numel():
         q = rotate_pairs_first(q, positions[:t], inv_freq, rot_scale, interleaved)
         k = rotate_pairs_first(k, positions[:t], inv_freq, rot_scale, interleaved)
-    q, k = rms_norm_to(q, q_norm, eps, torch.float32), rms_norm_to(k, k_norm, eps, torch.float32)
+    if normed:
+        q, k = rms_norm_to(q, q_norm, eps, torch.float32), rms_norm_to(k, k_norm, eps, torch.float32)
     if k_cache is not None:
         v = x[:, qs + ks:qs + ks + num_kv_heads * vdim].reshape(t, num_kv_heads, vdim)
         bs = k_cache.shape[2]
@@ -1051,7 +1084,7 @@ def rotate_norm_cache(x: torch.Tensor, num_heads: int, num_kv_heads: int, dim: i
         blk, off = sm // bs, sm % bs
         k_cache[blk, :, off, :] = k[valid].to(k_cache.dtype)
         v_cache[blk, :, off // V_GROUP, :, off % V_GROUP] = v[valid].to(v_cache.dtype)
-    return q.to(x.dtype)
+    return q.to(dtype)
 
 
 def gelu_and_mul(x: torch.Tensor, tanh: bool = True) -> torch.Tensor:

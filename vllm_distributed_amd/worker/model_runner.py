@@ -329,10 +329,10 @@ class ModelRunner:
                                dtype_bytes=self.model_config.dtype_bytes, values_per_token=0,
                                state_bytes_per_request=self._state_bytes_per_slot())
         a = layers[0]
-        windows = [int(getattr(l, "window", 0) or 0) for l in layers]
+        windows = [int(getattr(l, "reach", 0) or 0) for l in layers]
         dtype_bytes = 1 if fp8 else self.model_config.dtype_bytes
         if self.draft is not None:        # the draft reads every key it ever wrote unless it is windowed too
-            windows += [int(getattr(l, "window", 0) or 0) for l in self.draft.model.attention_layers()]
+            windows += [int(getattr(l, "reach", 0) or 0) for l in self.draft.model.attention_layers()]
         heads, width = a.num_kv_heads, a.head_dim
         if getattr(a, "latent", False):
             # one shared latent row per token, held in two layouts: (rank + rope) + rank values, which the
