@@ -1,0 +1,840 @@
+"""Bapovik through the framework (loader, scheduler, block and state-slot bookkeeping, model runner, kernels on the
+GPU / reference ops on the CPU) against the plain float64 model of ``tests/bapovik_oracle.py``.
+
+Every test builds its own small configuration and random weights (stored as bfloat16, so the oracle and the framework
+read the same numbers).  The schedules go through ``EngineCore.step_forced`` and generation goes through
+``LLM.generate``.  The CPU tests run in float32; the GPU tests run the HIP kernels in float32 (tight tolerance: an index
+that is one off shows) and in bfloat16 (with routers made decisive, see ``model_dir``).
+"""
+import json
+import math
+import os
+import types
+
+import numpy as np
+import pytest
+import torch
+
+import bapovik_oracle as oracle
+from test_tavulix import portions, run_schedule, tokens_for
+
+F64 = torch.float64
+
+
+# ------------------------------------------------------------------------------------------------ models
+def moe(experts, top, ff):
+    return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+
+
+def attention(heads, kv, dim, vdim, window, mlp=None, kv_from=None, scale=None):
+    m = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "mask": {"size": window},
+         "scale": dim ** -0.5 if scale is None else scale}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def parallel(left, right, mlp=None):
+    """``left``: heads, kv heads, dim, vdim, chunk, score scale, cap; ``right``: heads, dim, vdim, tau."""
+    lh, lk, ld, lv, chunk, scale, cap = left
+    rh, rd, rv, tau = right
+    return {"type": "parallel", "mlp": mlp,
+            "mixer": {"left": {"heads": lh, "kv_heads": lk, "dim": ld, "vdim": lv, "mask": {"size": chunk}, "scale": scale,
+                               "softcap": cap},
+                      "right": {"heads": rh, "dim": rd, "vdim": rv, "tau": tau}}}
+
+
+def config(layers, width=48, vocab=97, eps=1e-5):
+    return {"architecture": "Bapovik", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
+
+
+CONFIGS = {
+    # every layer of another shape and kind, attention first; query heads sharing key heads; key and value sizes that
+    # differ; two layers reading one layer's keys, through a wider and a narrower window, another owner of
+    # the same shape between them
+    "varied": config([
+        attention(4, 2, 8, 12, 9, moe(5, 2, 24)),
+        parallel((4, 2, 16, 12, 11, 0.9, 4.0), (3, 8, 20, 16.0), moe(4, 1, 16)),
+        attention(4, 2, 8, 12, 23, moe(3, 3, 40), kv_from=0),
+        parallel((3, 1, 8, 20, 25, 1.7, 1.5), (2, 24, 12, 3.0)),
+        attention(4, 2, 8, 12, 7),
+        attention(4, 2, 8, 12, 4, None, kv_from=0, scale=0.8),
+        attention(2, 1, 20, 8, 14, moe(6, 2, 8))]),
+    # values a model can make equal or one: one head, kv heads = heads, one expert, rank one, a window and a chunk of one
+    # token, masks wider than the text, tau and scale of one
+    "degenerate": config([
+        parallel((1, 1, 16, 16, 1, 1.0, 1.0), (1, 1, 1, 1.0), moe(1, 1, 8)),
+        attention(1, 1, 8, 8, 1, moe(2, 2, 4)),
+        attention(2, 2, 8, 8, 500),
+        parallel((2, 2, 8, 8, 400, 1.0, 30.0), (1, 8, 8, 1.0), moe(2, 1, 16)),
+        attention(2, 2, 8, 8, 1, None, kv_from=2)], width=32, vocab=50),
+    # masks and sequences over several pages of 16 tokens
+    "paged": config([
+        parallel((4, 1, 16, 16, 40, 1.1, 6.0), (4, 16, 16, 8.0), moe(8, 2, 32)),
+        attention(4, 4, 16, 24, 33, moe(4, 1, 32)),
+        attention(4, 4, 16, 24, 49, moe(4, 2, 16), kv_from=1),
+        parallel((2, 2, 32, 24, 48, 0.8, 20.0), (2, 20, 32, 16.0))], width=64),
+    # sizes the 16-bit kernels' 16-byte and matrix-core paths take
+    "wide": config([
+        attention(8, 2, 32, 64, 40, moe(6, 2, 128)),
+        parallel((4, 2, 64, 64, 37, 0.7, 8.0), (4, 32, 64, 4.0), moe(5, 1, 64)),
+        attention(8, 2, 32, 64, 21, moe(4, 2, 64), kv_from=0),
+        parallel((8, 2, 32, 32, 64, 1.0, 3.0), (1, 128, 32, 16.0))], width=128),
+    # a width, a vocabulary and sizes that are no multiples of 8 (no 16-byte access fits a 16-bit row)
+    "uneven": config([
+        parallel((3, 3, 20, 10, 18, 0.9, 2.0), (3, 10, 14, 5.0), moe(3, 2, 26)),
+        attention(3, 1, 12, 20, 13, moe(5, 1, 30)),
+        attention(3, 1, 12, 20, 30, None, kv_from=1)], width=100, vocab=211),
+    # no recurrence anywhere: no state slots at all
+    "windows": config([attention(2, 1, 16, 16, 12, moe(3, 1, 16)), attention(2, 1, 16, 16, 31, None, kv_from=0)], width=40),
+}
+RANKS = {"varied": 5, "degenerate": 1, "paged": 16, "wide": 24, "uneven": 3, "windows": 1}
+
+
+def random_weights(cfg, seed, rank):
+    g = torch.Generator().manual_seed(seed)
+    width = cfg["width"]
+
+    def rnd(*shape, lo=-1.0, hi=1.0):
+        return lo + (hi - lo) * torch.rand(shape, generator=g)
+
+    def proj(rows, cols, gain=1.0):
+        return rnd(rows, cols) * gain * (3.0 / cols) ** 0.5
+
+    def heads_of(q, m, own):
+        heads, kv, dim, vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        for nm, rows in (("q", heads * dim),) + ((("k", kv * dim), ("v", kv * vdim)) if own else ()):
+            w[q + nm], w[q + nm + ".b"] = proj(rows, width, 1.5 if nm == "q" else 1.0), rnd(rows, lo=-0.5, hi=0.5)
+        w[q + "g"], w[q + "o"] = proj(heads, width, 2.0), proj(width, heads * vdim, 1.5)
+
+    w = {"embed": rnd(cfg["vocab"], width), "head": proj(cfg["vocab"], width), "final.norm": rnd(width, lo=0.6, hi=1.4)}
+    for i, spec in enumerate(cfg["layers"]):
+        m, p = spec["mixer"], f"l{i}."
+        w[p + "norm1"] = rnd(width, lo=0.6, hi=1.4)
+        if spec["type"] == "attention":
+            heads_of(p + "mix.", m, "kv_from" not in m)
+        else:
+            q = p + "mix.left."
+            heads_of(q, m["left"], True)
+            for nm in ("q", "k"):
+                w[q + nm + ".norm"] = rnd(m["left"]["dim"], lo=0.6, hi=1.4)
+            w[q + "out"] = rnd(width, lo=0.6, hi=1.4)
+            r, q = m["right"], p + "mix.right."
+            heads, dim, vdim = r["heads"], r["dim"], r["vdim"]
+            for nm, rows in (("q", heads * dim), ("k", heads * dim), ("v", heads * vdim), ("g", heads * vdim)):
+                w[q + nm] = proj(rows, width)
+            w[q + "a1"], w[q + "a2"], w[q + "a2.b"] = proj(rank, width), proj(heads * dim, rank, 2.0), rnd(heads * dim, lo=-2.0, hi=3.0)
+            w[q + "norm"], w[q + "out"], w[q + "o"] = rnd(vdim, lo=0.6, hi=1.4), rnd(width, lo=0.6, hi=1.4), proj(width, heads * vdim)
+        if spec["mlp"]:
+            ff, experts = spec["mlp"]["expert"]["ff"], spec["mlp"]["router"]["experts"]
+            w[p + "mlp.router"] = proj(experts, width, 1.5)
+            for e in range(experts):
+                w[f"{p}mlp.e{e}.up"], w[f"{p}mlp.e{e}.down"] = proj(ff, width, 1.3), proj(width, ff)
+    return {k: v.to(torch.bfloat16) for k, v in w.items()}
+
+
+_MODELS, _ORACLE = {}, {}
+
+
+def save_model(d, cfg, w):
+    from safetensors.torch import save_file
+    save_file({k: v.contiguous() for k, v in w.items()}, str(d / "model.safetensors"))
+    (d / "config.json").write_text(json.dumps(cfg))
+    return str(d)
+
+
+def model_dir(name, tmp_path_factory, dtype="float32"):
+    """The model's folder, configuration and weights.  For bfloat16 runs the routers are made decisive: coordinate 0 of every
+    token vector is 3 or -3, no mixer or expert writes to it, and every router reads that coordinate only, with multipliers
+    1.5 apart in a random order.  The order of the scores is then a matter of the token whatever rounding does to the logits,
+    while the scores, which are the weights, still differ from row to row.  In bfloat16 the router's input carries the
+    rounding of every layer before it, and a close call that falls the other way swaps a whole expert; the float32 runs keep
+    the free-running routers."""
+    decisive = dtype != "float32"
+    if (name, decisive) not in _MODELS:
+        cfg = CONFIGS[name]
+        w = random_weights(cfg, sum(map(ord, name)), RANKS[name])
+        if decisive:
+            g = torch.Generator().manual_seed(11)
+            w["embed"][:, 0] = 3.0 * (2.0 * torch.randint(0, 2, (cfg["vocab"],), generator=g) - 1.0)
+            for k in list(w):
+                if k.endswith(".out") or (k.endswith(".o") and ".left." not in k and ".right." not in k) or k.endswith(".down"):
+                    w[k][0] = 0.0
+                if k.endswith(".router"):
+                    experts = w[k].shape[0]
+                    w[k] = torch.zeros_like(w[k])
+                    w[k][:, 0] = ((torch.randperm(experts, generator=g).float() - (experts - 1) / 2) * 1.5).to(torch.bfloat16)
+                if k.endswith("norm1"):
+                    w[k][0] = 1.0
+        d = tmp_path_factory.mktemp("bapovik_" + name)
+        _MODELS[(name, decisive)] = (save_model(d, cfg, w), cfg, w)
+    return _MODELS[(name, decisive)]
+
+
+def oracle_logits(cfg, w, tokens, single=False):
+    """The float64 model's logits; ``single``: the same equations evaluated in float32."""
+    key = (id(w), tuple(tokens), single)
+    if key not in _ORACLE:
+        kind = torch.float32 if single else torch.float64
+        saved = oracle.F64, oracle.f64
+        oracle.F64, oracle.f64 = kind, (lambda t: t.to(kind))
+        try:
+            # (the weights are kept with the result: their identity is the key)
+            _ORACLE[key] = (w, oracle.forward(cfg, w, list(tokens)).double().numpy())
+        finally:
+            oracle.F64, oracle.f64 = saved
+    return _ORACLE[key][1]
+
+
+def check(got, cfg, w, reqs, tol):
+    """Every row the run produced against the oracle.  Both halves of a parallel mixer and every recurrent head are normed, so
+    at a position where an output nearly cancels, the rounding of its inputs is multiplied up.  How much a row multiplies
+    rounding is measured, not guessed: the oracle's own equations evaluated in float32 differ from float64 by some ``e32``
+    at that row (a few 1e-6 where nothing cancels), and the row is allowed ``8 e32`` in float32 and ``2^14 e32`` in bfloat16
+    where that is more than the tolerance.  A wrong index or a lost state shows in many rows, none of them of that kind."""
+    assert got
+    room = 8.0 if tol < 1e-2 else 16384.0
+    over = []
+    for (rid, p), row in got.items():
+        want = oracle_logits(cfg, w, reqs[rid])[p]
+        e32 = float(np.abs(oracle_logits(cfg, w, reqs[rid], single=True)[p] - want).max())
+        ratio = float(np.abs(row - want).max()) / max(tol, room * e32)
+        if not ratio <= 1.0:
+            over.append((ratio, rid, p, e32))
+    over.sort(reverse=True)
+    # (in bfloat16 a row in fifty may lie outside, by a factor of three at most: the tolerance is a typical worst row)
+    assert not over or (tol > 1e-2 and over[0][0] <= 3.0), over[:5]
+    assert len(over) <= max(1, len(got) // 50), over[:5]
+
+
+DEVICES = [pytest.param("cpu", "float32", 1e-4, id="cpu-f32"),
+           pytest.param("cuda", "float32", 1e-4, id="gpu-f32", marks=pytest.mark.gpu),
+           pytest.param("cuda", "bfloat16", 0.2, id="gpu-bf16", marks=pytest.mark.gpu)]
+OP_DEVICES = [pytest.param("cpu", "float32", id="cpu-f32"),
+              pytest.param("cuda", "float32", id="gpu-f32", marks=pytest.mark.gpu),
+              pytest.param("cuda", "bfloat16", id="gpu-bf16", marks=pytest.mark.gpu)]
+
+
+def i32(device, *values):
+    return torch.tensor(list(values), dtype=torch.int32, device=device)
+
+
+# ------------------------------------------------------------------------------------------------ schedules
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_whole_prompt_and_first_tokens(name, device, dtype, tol, tmp_path_factory, tmp_path):
+    path, cfg, w = model_dir(name, tmp_path_factory, dtype)
+    reqs = {"a": tokens_for(cfg, 110, 1), "b": tokens_for(cfg, 1, 2), "c": tokens_for(cfg, 2, 3)}
+    steps = [[(r, t, list(range(len(t)))), {"end": [r]}] for r, t in reqs.items()]
+    got = run_schedule(path, steps, dtype, device, max_tokens=128, tmp=tmp_path)
+    assert len(got) == 113
+    check(got, cfg, w, reqs, tol)
+
+
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+@pytest.mark.parametrize("name", ["varied", "uneven"])
+def test_residual_stream_after_every_layer(name, device, dtype, tol, tmp_path_factory):
+    if dtype != "float32":
+        pytest.skip("the per-layer comparison is the float32 one")
+    from vllm_distributed_amd.engine.request import Request
+    from vllm_distributed_amd.entrypoints import trace_replay
+    from vllm_distributed_amd.sampling_params import SamplingParams
+    path, cfg, w = model_dir(name, tmp_path_factory)
+    toks = tokens_for(cfg, 37, 8)
+    args = types.SimpleNamespace(model=path, dtype=dtype, out="", max_tokens=64, max_seqs=2, device=device,
+                                 block_size=16, enforce_eager=True)
+    core = trace_replay.make_core(args)
+    try:
+        model = core.executor.driver.worker.model_runner.model
+        model.trace_residual = []
+        core.add_request(Request("r", toks, SamplingParams(temperature=0.0, max_tokens=None, score_only=True, ignore_eos=True)))
+        core.step_forced({"r": len(toks)}, {})
+        got = [t.cpu().double() for t in model.trace_residual]
+    finally:
+        core.shutdown()
+    want = []
+    oracle.forward(cfg, w, toks, want)
+    assert len(got) == len(want) == len(cfg["layers"])
+    for i, (a, b) in enumerate(zip(got, want)):
+        assert (a - b).abs().max().item() <= 2e-5 * max(1.0, b.abs().max().item()), i
+
+
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+@pytest.mark.parametrize("name", ["varied", "paged", "wide", "windows"])
+def test_prefill_then_long_token_by_token_decoding(name, device, dtype, tol, tmp_path_factory, tmp_path):
+    """A prompt, then 120 tokens one at a time: every window and every chunk passes over decoded tokens, the recurrent
+    state is carried through 120 single-row steps, the cache grows over several pages."""
+    path, cfg, w = model_dir(name, tmp_path_factory, dtype)
+    toks = tokens_for(cfg, 150, 4)
+    got = run_schedule(path, portions(toks, [30, 1], "r"), dtype, device, max_tokens=192, tmp=tmp_path)
+    assert len(got) == 150
+    check(got, cfg, w, {"r": toks}, tol)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype,tol", [("float32", 1e-4), ("bfloat16", 0.2)])
+@pytest.mark.parametrize("name", ["paged", "wide"])
+def test_pages_of_64_tokens(name, dtype, tol, tmp_path_factory, tmp_path):
+    """The page size a GPU engine uses by default: two requests in turn, portions that end inside, at and just
+    behind a page's border, then single rows across the next border."""
+    path, cfg, w = model_dir(name, tmp_path_factory, dtype)
+    a, b = tokens_for(cfg, 150, 60), tokens_for(cfg, 70, 61)
+    steps = [[("a", a[:63], [0, 62])], [("a", a[63:64], [0]), ("b", b[:64], [63])], [("a", a[64:66], [0, 1]), ("b", b[64:65], [0])],
+             [("a", a[66:127], [60]), ("b", b[65:70], [4]), {"end": ["b"]}]]
+    steps += [[("a", a[i:i + 1], [0])] for i in range(127, 150)]
+    steps[-1].append({"end": ["a"]})
+    got = run_schedule(path, steps, dtype, "cuda", max_tokens=256, block_size=64, tmp=tmp_path)
+    assert len(got) == 2 + 1 + 1 + 2 + 1 + 1 + 1 + 23
+    check(got, cfg, w, {"a": a, "b": b}, tol)
+
+
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+@pytest.mark.parametrize("sizes", [[2], [3, 2, 7, 1, 16, 17, 2, 2, 31, 5], [1], [64, 2, 1]])
+@pytest.mark.parametrize("name", ["varied", "wide"])
+def test_portions_of_any_size(name, sizes, device, dtype, tol, tmp_path_factory, tmp_path):
+    """Portions cut inside pages, windows and chunks (the mask's and the recurrence kernel's), down to two tokens and one."""
+    path, cfg, w = model_dir(name, tmp_path_factory, dtype)
+    toks = tokens_for(cfg, 85 if sizes != [1] else 40, 5)
+    got = run_schedule(path, portions(toks, sizes, "r"), dtype, device, max_tokens=128, tmp=tmp_path)
+    assert len(got) == len(toks)
+    check(got, cfg, w, {"r": toks}, tol)
+
+
+def unequal_requests(cfg):
+    """Seven unequal requests for three sequence slots and 10 pages of 16: portions of prompts beside single tokens,
+    requests that sit steps out, slots and pages handed on as requests end."""
+    reqs = {f"q{i}": tokens_for(cfg, n, 10 + i) for i, n in enumerate([50, 33, 1, 47, 20, 48, 9])}
+    at = {r: 0 for r in reqs}
+    pattern = {"q0": [7, 1, 1, 2, 30, 1], "q1": [2, 16, 1, 1, 1], "q2": [1], "q3": [17, 1, 15, 1], "q4": [1, 1, 5],
+               "q5": [30, 2, 1], "q6": [2, 1]}
+    waiting, live, steps, turn = list(reqs), [], [], 0
+    while waiting or live:
+        while waiting and len(live) < 3 and \
+                sum(-(-len(reqs[r]) // 64) * 64 for r in live + waiting[:1]) <= 160:
+            live.append(waiting.pop(0))
+        step, ended = [], []
+        for k, r in enumerate(list(live)):
+            if (turn + k) % 4 == 3 and len(live) > 1:
+                continue                                    # sits this step out
+            sizes = pattern[r]
+            n = min(sizes[min(at[r] and (turn % len(sizes)), len(sizes) - 1)], len(reqs[r]) - at[r])
+            step.append((r, reqs[r][at[r]:at[r] + n], list(range(n))))
+            at[r] += n
+            if at[r] == len(reqs[r]):
+                ended.append(r)
+                live.remove(r)
+        if step:
+            steps.append(step + ([{"end": ended}] if ended else []))
+        turn += 1
+    return reqs, steps
+
+
+@pytest.mark.parametrize("eager", [False, True])
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+@pytest.mark.parametrize("name", ["paged", "wide", "windows"])
+def test_mixed_batches_reuse_pages_and_slots(name, device, dtype, tol, eager, tmp_path_factory, tmp_path):
+    """A new owner of a page or slot must not see what the old one left; every row against the request run alone by the
+    oracle."""
+    if eager and device == "cpu":
+        pytest.skip("graphs exist on the GPU only")
+    path, cfg, w = model_dir(name, tmp_path_factory, dtype)
+    reqs, steps = unequal_requests(cfg)
+    got = run_schedule(path, steps, dtype, device, max_tokens=160, max_seqs=3, eager=eager, tmp=tmp_path)
+    assert len(got) == sum(len(t) for t in reqs.values())
+    check(got, cfg, w, reqs, tol)
+
+
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+def test_batch_rows_equal_single_runs(device, dtype, tol, tmp_path_factory, tmp_path):
+    """The same rows run alone and inside a batch of unequal neighbours agree far inside the oracle tolerance."""
+    path, cfg, w = model_dir("varied", tmp_path_factory, dtype)
+    a, b, c = tokens_for(cfg, 30, 20), tokens_for(cfg, 11, 21), tokens_for(cfg, 64, 22)
+    alone = run_schedule(path, portions(a, [13, 1], "a"), dtype, device, max_tokens=64, tmp=tmp_path / "x")
+    steps = [[("c", c[:50], []), ("a", a[:13], list(range(13))), ("b", b[:2], [])]]
+    for i in range(13, 30):
+        step = [("a", a[i:i + 1], [0])]
+        if i < 22:
+            step.append(("b", b[i - 11:i - 10], []))
+        if i < 27:
+            step.insert(0, ("c", c[50 + i - 13:51 + i - 13], []))
+        steps.append(step)
+    both = run_schedule(path, steps, dtype, device, max_tokens=192, tmp=tmp_path / "y")
+    worst = sorted(float(np.abs(alone[("a", p)] - both[("a", p)]).max()) for p in range(30))
+    assert worst[-1 if dtype == "float32" else -2] <= (5e-5 if dtype == "float32" else 0.12), worst[-3:]
+
+
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+def test_a_reader_that_looks_further_back_than_the_owner(device, dtype, tol, tmp_path_factory, tmp_path):
+    """A layer with a window of 8 owns the keys, another reads them through a window of 260: the pages stay with the request
+    as long as the WIDEST reader looks at them.  A long request decodes while short ones come and go on what pages the pool
+    has left; given back too early, its pages would be written over."""
+    cfg = config([attention(2, 1, 16, 16, 8), attention(2, 1, 16, 16, 260, None, kv_from=0),
+                  parallel((2, 1, 8, 8, 20, 1.0, 5.0), (1, 8, 8, 4.0))], width=40, vocab=60)
+    w = random_weights(cfg, 21, 4)
+    d = tmp_path_factory.mktemp("bapovik_reader")
+    path = save_model(d, cfg, w)
+    reqs = {"a": tokens_for(cfg, 440, 30), **{f"s{i}": tokens_for(cfg, 60, 31 + i) for i in range(6)}}
+    steps = [[("a", reqs["a"][:290], [289])]]
+    at = 290
+    for i in range(6):
+        for lo, hi in ((0, 33), (33, 34), (34, 60)):
+            n = 8
+            steps.append([("a", reqs["a"][at:at + n], list(range(n))), (f"s{i}", reqs[f"s{i}"][lo:hi], [hi - lo - 1])])
+            at += n
+        steps[-1].append({"end": [f"s{i}"]})
+    steps += [[("a", reqs["a"][k:k + 1], [0])] for k in range(at, 440)]
+    steps[-1].append({"end": ["a"]})
+    got = run_schedule(path, steps, dtype, device, max_tokens=512, tmp=tmp_path)
+    assert len(got) == 1 + 150 + 18
+    check(got, cfg, w, reqs, tol)
+
+
+@pytest.mark.parametrize("device,dtype,tol", DEVICES)
+def test_one_far_token_decides_the_logits(device, dtype, tol, tmp_path_factory, tmp_path):
+    """Models whose attention can be aimed: the queries of one layer read a coordinate of the embedding that only one token
+    has, its keys one that only another token has, and that key's value marks the logits - exactly when the mask lets it be seen.
+    Window (own keys and another layer's), chunk; the far token just inside and just outside, at page borders; the asking
+    token in the prompt, at a portion's start and decoded alone."""
+    width, dim = 64, 32
+    window, chunk, reader = 70, 50, 101
+    for kind, reach in (("window", lambda i, j: i - j < window), ("reader", lambda i, j: i - j < reader),
+                        ("chunk", lambda i, j: i // chunk == j // chunk)):
+        aimed = {"window": [attention(2, 1, dim, 16, window, None, None, 1.0)],
+                 "reader": [attention(2, 1, dim, 16, 3, None, None, 0.01), attention(2, 1, dim, 16, reader, None, 0, 1.0)],
+                 "chunk": [parallel((2, 1, dim, 16, chunk, 1.0, 40.0), (1, 8, 8, 4.0))]}[kind]
+        cfg = config(aimed, width=width, vocab=80)
+        w = {k: v.float() for k, v in random_weights(cfg, 5, 4).items()}
+        g = torch.Generator().manual_seed(6)
+        w["embed"][:, :4] = 0.02 * torch.randn(80, 4, generator=g)
+        w["embed"][78, 0], w["embed"][79, 2] = 6.0, 6.0              # 78: the far token, 79: the one that asks for it
+        w["embed"][78, 1] = 4.0                                      # what the far token's value carries
+        at = f"l{len(aimed) - 1}.mix." + ("left." if kind == "chunk" else "")
+        own = "l0.mix." + ("left." if kind == "chunk" else "")
+        if kind == "reader":                                         # the owner itself passes nothing on
+            w["l0.mix.o"] *= 0.0
+        for name, c in ((at + "q", 2), (own + "k", 0)):
+            m = 0.02 * torch.randn(w[name].shape, generator=g)
+            m[3::dim, c] = 3.0
+            w[name] = m
+            w[name + ".b"] *= 0.0
+            if kind == "chunk":
+                w[name + ".norm"] = torch.ones(dim)
+                w[name][5::dim, 7] = 1.0                             # (other tokens' heads have another direction)
+                w["embed"][:78, 7] = 2.0
+        v = 0.1 * torch.randn(w[own + "v"].shape, generator=g)
+        v[:, 1] = torch.linspace(1.0, 3.0, 16)
+        w[own + "v"] = v
+        w = {k: x.to(torch.bfloat16) for k, x in w.items()}
+        path = save_model(tmp_path_factory.mktemp("bapovik_far_" + kind), cfg, w)
+        base = [int(t) % 78 for t in tokens_for(cfg, 270, 9)]
+        edge = {"window": window, "reader": reader, "chunk": None}[kind]
+        cases = ([(100, 149, 149), (100, 149, 120), (99, 149, 149), (99, 100, 100), (112, 113, 64), (150, 199, 190), (149, 150, 150),
+                  (0, 49, 30), (49, 50, 50)] if kind == "chunk" else
+                 [(200 - edge + 1, 200, 200), (200 - edge, 200, 200), (200 - edge + 1, 200, 150), (200 - edge, 200, 150),
+                  (160, 160 + edge - 1, 160), (144, 144 + edge, 144 + edge), (15, 60, 16), (0, edge - 1, 32), (0, edge, edge)])
+        seen_both = set()
+        for far, late, cut in cases:
+            toks = list(base)
+            toks[far], toks[late] = 78, 79
+            steps = [[("r", toks[:cut], [0])]] if cut == late else [[("r", toks[:cut], [0])], [("r", toks[cut:late], [0])]]
+            steps += [[("r", toks[late:late + 1], [0]), {"end": ["r"]}]]
+            steps += [[("s", toks[:late + 1], [late]), {"end": ["s"]}]]
+            got = run_schedule(path, steps, dtype, device, max_tokens=320, tmp=tmp_path)
+            want = oracle_logits(cfg, w, toks[:late + 1])[late]
+            blank = list(toks)
+            blank[far] = 3
+            shows = np.abs(want - oracle_logits(cfg, w, blank[:late + 1])[late]).max()
+            seen = reach(late, far)
+            seen_both.add(seen)
+            assert (shows > 0.4) == seen, (kind, far, late, shows)   # (the far token decides, or it is not seen at all)
+            for key in (("r", late), ("s", late)):
+                assert np.abs(got[key] - want).max() < (1e-4 if dtype == "float32" else 0.1), (kind, far, late, key)
+        assert seen_both == {True, False}
+
+
+# --------------------------------------------------------------------------- mechanisms alone, made to show
+@pytest.mark.parametrize("device,dtype", OP_DEVICES)
+@pytest.mark.parametrize("dim,vdim", [(8, 12), (32, 16), (64, 64), (20, 40)])
+@pytest.mark.parametrize("chunked", [False, True])
+def test_one_key_stands_out_at_every_edge(device, dtype, dim, vdim, chunked):
+    """Attention as the layers run it, over shuffled pages, one key far above all others: it gets its whole share exactly when
+    the mask shows it - first and last token of the window or chunk, the ones next to them, page borders, the row itself, a
+    key behind the row.  Capped scores: the share is ``e^(cap tanh(s / cap)) / (open + e^..)`` in closed form, with one in
+    the denominator (chunked) or without; the head's gate multiplies it; pages wholly out of sight are poisoned."""
+    from vllm_distributed_amd.models.layers.attention import AttentionMetadata, WindowBiasAttention, set_forward_context
+    dt = getattr(torch, dtype)
+    n, bs, hq, hkv, size, cap = 250, 16, 4, 2, 40, 3.0
+    g = torch.Generator().manual_seed(dim)
+    nblk = -(-n // bs) + 2
+    table = torch.randperm(nblk, generator=g)[:-(-n // bs)].to(torch.int32).view(1, -1)
+    with torch.device(device):
+        owner = WindowBiasAttention(hq, dim, vdim, hkv, 1.0, 0, window=5, distance_bias=False, sink=False)
+        attn = (WindowBiasAttention(hq, dim, vdim, hkv, 0.5, 0, chunk=size, softcap=cap, distance_bias=False, sink=0.0)
+                if chunked else
+                WindowBiasAttention(hq, dim, vdim, hkv, 0.5, 1, window=size, distance_bias=False, sink=False, source=owner))
+    assert owner.reach == (5 if chunked else size) and attn.window == size
+    vals = torch.randn(n, hkv, vdim, generator=g)
+    gate = torch.tensor([[0.4, -1.0, 2.0, 0.0]])
+
+    def run(target, q, pos, rows):
+        kc = torch.zeros(nblk, hkv, bs, dim, dtype=dt)
+        vc = torch.zeros(nblk, hkv, bs // 8, vdim, 8, dtype=dt)
+        for j in range(n):
+            b, o = int(table[0, j // bs]), j % bs
+            kc[b, :, o, 0] = 0.0 if j == target else -80.0     # everything else far below
+            kc[b, :, o, 1] = 1.0 if j == target else 0.0
+            vc[b, :, o // 8, :, o % 8] = vals[j].to(dt)
+        first = pos - rows + 1
+        lo = first // size * size if chunked else max(first - size + 1, 0)
+        # (the kernels fetch whole tiles of 32 keys; the plain form multiplies hidden values by zero)
+        bad = float("nan") if device == "cuda" else 1e4
+        for blk in range((lo & ~31) // bs):
+            kc[table[0, blk]], vc[table[0, blk]] = bad, bad
+        (attn if chunked else owner).bind_kv_cache(kc.to(device), vc.to(device))
+        qsl = i32(device, 0, rows)
+        md = AttentionMetadata(num_decodes=1 if rows == 1 else 0, num_decode_tokens=1 if rows == 1 else 0,
+                               num_prefills=0 if rows == 1 else 1, num_prefill_tokens=0 if rows == 1 else rows,
+                               slot_mapping=i32(device, *([-1] * rows)), block_table=table.to(device),
+                               seq_lens=i32(device, pos + 1), query_start_loc=qsl, max_query_len=rows, max_seq_len=pos + 1,
+                               prefill_query_start_loc=qsl, max_prefill_query_len=rows)
+        set_forward_context(md, torch.arange(first, pos + 1, dtype=torch.int32, device=device))
+        try:
+            o = attn.forward_cached(q.to(dt).to(device), gate.repeat(rows, 1).to(dt).to(device)).view(rows, hq, vdim)
+            return o[-1].float().cpu()
+        finally:
+            set_forward_context(None)
+    for pos in (249, 240, 239, 200, 120, 119, 40, 39, 16, 0):
+        lo = pos // size * size if chunked else max(pos - size + 1, 0)
+        for target in sorted({lo, lo + 1, lo - 1, pos, pos - 1, pos // bs * bs, pos // bs * bs - 1, pos + 1}):
+            if target < 0 or target >= n:
+                continue
+            for rows in (1, min(9, pos + 1)):
+                q = torch.zeros(rows, hq, dim)
+                q[:, :, 0] = 1.0
+                q[-1, :, 1] = torch.tensor([-1.0, 0.0, 2.0, 6.0])
+                o = run(target, q, pos, rows)
+                seen = lo <= target <= pos
+                for h in range(hq):
+                    s, rest = 0.5 * float(q[-1, h, 1]), -40.0
+                    if chunked:
+                        s, rest = cap * math.tanh(s / cap), cap * math.tanh(-40.0 / cap)
+                    own = math.exp(s) if seen else 0.0
+                    others = [j for j in range(lo, pos + 1) if j != target]
+                    total = own + len(others) * math.exp(rest) + (1.0 if chunked else 0.0)
+                    vd = vals[:, h // 2].to(dt).float()
+                    want = (own * vd[target] + math.exp(rest) * vd[others].sum(0)) / total
+                    want = want / (1.0 + math.exp(-float(gate[0, h])))
+                    if not chunked and not seen:
+                        want = vd[others].mean(0) / (1.0 + math.exp(-float(gate[0, h])))
+                    assert (o[h] - want).abs().max().item() < (2e-5 if dtype == "float32" else 0.03), (pos, target, rows, h)
+
+
+@pytest.mark.parametrize("device,dtype", OP_DEVICES)
+@pytest.mark.parametrize("heads,dim,vdim,tau", [(2, 8, 12, 16.0), (1, 64, 64, 4.0), (3, 20, 6, 1.0), (1, 160, 32, 16.0)])
+def test_channels_decay_by_themselves_and_stale_slots_do_not_show(device, dtype, heads, dim, vdim, tau):
+    """Token 0 writes along two key channels nobody else touches, one that keeps and one that forgets; 300 tokens later the
+    query reads both: what the first channel's decays left of the value, nothing of the second's.  Decays come from the
+    rows through the narrow projection.  Portions of many sizes through a slot another sequence left full; the whole against
+    the token-by-token float64 recurrence."""
+    from vllm_distributed_amd import ops
+    dt = getattr(torch, dtype)
+    n, rank, keep, forget = 301, 3, 2, 5
+    g = torch.Generator().manual_seed(dim)
+    q, k = torch.randn(n, heads, dim, generator=g), torch.randn(n, heads, dim, generator=g)
+    v = 0.1 * torch.randn(n, heads, vdim, generator=g)
+    k[:, :, [keep, forget]], q[n - 1] = 0.0, 0.0
+    k[0, :, [keep, forget]], q[n - 1, :, [keep, forget]], v[0] = 2.0, 1.0, 3.0
+    k[0, :, forget] = -2.0
+    a = torch.randn(n, rank, generator=g)
+    a2 = torch.randn(heads * dim, rank, generator=g)
+    bias = torch.randn(heads * dim, generator=g)
+    a2.view(heads, dim, rank)[:, [keep, forget]] = 0.0
+    bias.view(heads, dim)[:, keep], bias.view(heads, dim)[:, forget] = 5.0, -3.0 * tau
+    x = torch.cat([q.reshape(n, -1), k.reshape(n, -1), v.reshape(n, -1)], 1).to(dt)
+    a, a2 = a.to(dt), a2.to(dt)
+    xd = x.double()
+    alpha = (oracle.sigmoid(a.double() @ a2.double().T + bias.double()) ** (1.0 / tau)).view(n, heads, dim)
+    qs, hd = heads * dim, heads * dim
+    want, last = oracle.decayed_heads(xd[:, :qs].view(n, heads, dim) * dim ** -0.5, xd[:, qs:qs + hd].view(n, heads, dim),
+                                      xd[:, 2 * hd:].view(n, heads, vdim), alpha)
+    left = 2.0 * 3.0 * dim ** -0.5 * (1.0 / (1.0 + math.exp(-5.0))) ** (300 / tau)
+    assert (want[n - 1] - left).abs().max().item() < 0.02 * left
+    state = torch.full((3, heads, dim, vdim), 7.0, device=device)                  # what an earlier owner left
+    out, at, sizes = [], 0, [1, 2, 64, 17, 1, 1, 100, 3, 2, 16]
+    for i in range(100):
+        m = min(sizes[i % len(sizes)], n - at)
+        if m == 0:
+            break
+        al = ops.low_rank_decay(a[at:at + m].to(device), a2.to(device), bias.to(device), tau)
+        out.append(ops.decay_linear_attention(x[at:at + m].to(device), heads, dim, vdim, al, state, i32(device, 2),
+                                              i32(device, 0, m), i32(device, at + m), False, m, dim ** -0.5).cpu())
+        at += m
+    got = torch.cat(out).double().view(n, heads, vdim)
+    assert (got - want).abs().max().item() < 1e-5 * float(want.abs().max())
+    assert (state[2].cpu().double() - last).abs().max().item() < 1e-5 * float(last.abs().max())
+    assert float(state[0].min()) == 7.0 and float(state[1].max()) == 7.0
+
+
+@pytest.mark.parametrize("device", [pytest.param("cpu", id="cpu"), pytest.param("cuda", id="gpu", marks=pytest.mark.gpu)])
+def test_slow_decays_keep_their_precision(device):
+    """What a channel forgets per token, from a tenth down to one part in ten million, and decays of next to nothing."""
+    from vllm_distributed_amd import ops
+    z = torch.tensor([-60.0, -20.5, -19.5, -3.0, 0.0, 0.5, 3.0, 8.0, 11.0, 14.0])
+    for tau in (1.0, 16.0):
+        got = ops.low_rank_decay(torch.zeros(1, 1, device=device), torch.zeros(z.numel(), 1, device=device), z.to(device), tau)
+        want = oracle.sigmoid(z.double()) ** (1.0 / tau)
+        err = (got[0].cpu().double() - want).abs()
+        assert (err <= 1.3e-7 * torch.maximum(want, torch.tensor(1e-30, dtype=F64)) + 4e-6 * want * (want < 0.9)).all(), err
+
+
+@pytest.mark.parametrize("device,dtype", OP_DEVICES)
+def test_experts_weigh_their_input(device, dtype):
+    """One expert, one channel: the squared ReLU of a weighted input goes with the SQUARE of the weight (weighing the output
+    would go with the weight); scores are sigmoids as they come, several chosen experts are summed, not renormalised."""
+    from vllm_distributed_amd.models.layers.moe import PlainTopKMoE
+    dt = getattr(torch, dtype)
+    width = 128
+    with torch.device(device):
+        m = PlainTopKMoE(width, 64, 3, 2, dt, activation="relu2", scores="sigmoid", weigh_input=True)
+    for p in (m.w1, m.w2, m.gate.weight):
+        p.data.zero_()
+    m.gate.weight.data[:, 0] = torch.tensor([1.0, -0.5, -3.0])
+    m.w1.data[:, 0, 1] = torch.tensor([1.0, 2.0, 50.0])            # expert e's only inner channel reads coordinate 1
+    m.w2.data[:, 5, 0] = 1.0
+    for z in (0.5, -1.0, 3.0):
+        x = torch.zeros(4, width)
+        x[:, 0], x[0, 1], x[1, 1], x[2, 1], x[3, 1] = z, 2.0, -2.0, 0.5, 0.0
+        got = m(x.to(dt).to(device)).float().cpu()
+        logits = z * torch.tensor([1.0, -0.5, -3.0])
+        score = torch.sigmoid(logits.double())
+        chosen = sorted(torch.argsort(score, descending=True)[:2].tolist())
+        up = torch.tensor([1.0, 2.0, 50.0], dtype=F64)
+        for r in range(4):
+            want = sum(max(float(score[e] * up[e] * x[r, 1]), 0.0) ** 2 for e in chosen)
+            assert abs(float(got[r, 5]) - want) < (1e-6 if dtype == "float32" else 0.01) * max(want, 1.0), (z, r)
+        assert got[:, torch.arange(width) != 5].abs().max().item() == 0.0
+
+
+@pytest.mark.parametrize("device,dtype", OP_DEVICES)
+@pytest.mark.parametrize("hidden,ff,experts,top,rows", [(128, 96, 6, 2, 33), (256, 64, 9, 9, 5), (96, 40, 3, 1, 200), (64, 20, 1, 1, 7)])
+def test_expert_block_against_the_oracle(device, dtype, hidden, ff, experts, top, rows):
+    from vllm_distributed_amd.models.layers.moe import PlainTopKMoE
+    dt = getattr(torch, dtype)
+    g = torch.Generator().manual_seed(hidden)
+    w = {"router": torch.randn(experts, hidden, generator=g)}
+    for e in range(experts):
+        w[f"e{e}.up"] = torch.randn(ff, hidden, generator=g) * hidden ** -0.5
+        w[f"e{e}.down"] = torch.randn(hidden, ff, generator=g) * ff ** -0.5
+    x = torch.randn(rows, hidden, generator=g)
+    # one router row read per token by size: scores far apart
+    x[:, 0] = 1.0 + torch.rand(rows, generator=g)
+    w["router"] = torch.zeros(experts, hidden)
+    w["router"][:, 0] = torch.randperm(experts, generator=g).float() - experts / 2
+    w, x = {k: v.to(torch.bfloat16) for k, v in w.items()}, x.to(torch.bfloat16)
+    with torch.device(device):
+        m = PlainTopKMoE(hidden, ff, experts, top, dt, activation="relu2", scores="sigmoid", weigh_input=True)
+    m.gate.weight.data.copy_(w["router"])
+    for e in range(experts):
+        m._load_w1(m.w1, w[f"e{e}.up"], e)
+        m._load_w2(m.w2, w[f"e{e}.down"], e)
+    got = m(x.to(dt).to(device)).double().cpu()
+    want = oracle.experts(x.double(), w, "", {"router": {"top": top}})
+    assert (got - want).abs().max().item() < (1e-5 if dtype == "float32" else 0.02) * max(1.0, float(want.abs().max()))
+
+
+@pytest.mark.parametrize("device,dtype", OP_DEVICES)
+def test_halves_are_normed_before_they_meet(device, dtype):
+    """Half the sum of two normed outputs of very different size, a plain output beside them, and the norm of the sum that
+    the next layer reads: one call."""
+    from vllm_distributed_amd.models.layers.attention import ResidualRMSNorm
+    dt = getattr(torch, dtype)
+    g = torch.Generator().manual_seed(2)
+    width, eps = 72, 1e-5
+    with torch.device(device):
+        then = ResidualRMSNorm(width, eps, dt)
+    wy, wz, wn = (torch.rand(width, generator=g) + 0.5 for _ in range(3))
+    then.weight.data.copy_(wn)
+    x0 = 3 * torch.randn(5, width, generator=g)
+    size = torch.tensor([1e-4, 0.1, 1.0, 30.0, 300.0]).view(-1, 1)
+    y, z = (torch.randn(5, width, generator=g) * size).to(dt), (torch.randn(5, width, generator=g) * size.flip(0)).to(dt)
+    f = torch.randn(5, width, generator=g).to(dt)
+    for plain in (f, None):
+        want = x0.double() + 0.5 * (oracle.unit_rms(y.double(), eps) * wy.double() + oracle.unit_rms(z.double(), eps) * wz.double())
+        if plain is not None:
+            want = want + f.double()
+        x = x0.clone().to(device)
+        out = then.after_pair(y.to(device), wy.to(device), z.to(device), wz.to(device), 0.5,
+                              None if plain is None else plain.to(device), x)
+        assert (x.cpu().double() - want).abs().max().item() < 3e-6 and x.dtype == torch.float32
+        w2 = oracle.unit_rms(want, eps) * wn.double()
+        assert out.dtype == dt and (out.cpu().double() - w2).abs().max().item() < (1e-5 if dtype == "float32" else 0.05)
+
+
+# ------------------------------------------------------------------------------------------- bookkeeping
+def test_layers_caches_and_state(tmp_path_factory):
+    """Every layer with keys of its own owns cache rows, readers own none; every recurrent half an fp32 state and nothing
+    else; pages are kept as far back as the widest window, chunk or reader looks."""
+    from vllm_distributed_amd.entrypoints import trace_replay
+    path, cfg, w = model_dir("varied", tmp_path_factory)
+    args = types.SimpleNamespace(model=path, dtype="bfloat16", out="", max_tokens=64, max_seqs=3, device="cpu",
+                                 block_size=16, enforce_eager=True)
+    core = trace_replay.make_core(args)
+    try:
+        mr = core.executor.driver.worker.model_runner
+        owners = mr.model.attention_layers()
+        assert [a.layer_idx for a in owners] == [0, 1, 3, 4, 6]
+        assert [(a.window, a.chunk, a.reach) for a in owners] == [(9, 0, 23), (11, 11, 11), (25, 25, 25), (7, 0, 7),
+                                                                      (14, 0, 14)]
+        assert tuple(owners[0].k_cache.shape[1:]) == (2, 16, 8) and tuple(owners[0].v_cache.shape[1:]) == (2, 2, 12, 8)
+        readers = [mr.model.layers[i].mix.inner.attn for i in (2, 5)]
+        assert all(r.source is owners[0] and r.k_cache is None for r in readers) and [r.window for r in readers] == [23, 4]
+        assert [tuple(s.shape) for s in mr.state_tensors] == [(4, 3, 8, 20), (4, 2, 24, 12)]
+        assert all(s.dtype == torch.float32 for s in mr.state_tensors)
+        spec = mr.get_kv_cache_spec()
+        assert spec.sliding_window == 25 == core.kv_window
+        assert spec.bytes_per_token == 2 * (2 * 20 + 2 * 28 + 1 * 28 + 2 * 20 + 1 * 28)
+        names = [n for n, _ in mr.model.named_parameters()]
+        assert len(names) == len(set(names)) and "head.weight" in names
+    finally:
+        core.shutdown()
+
+
+def test_grouped_projection_starts_every_group_on_a_16_byte_border():
+    from vllm_distributed_amd.models.layers.linear import GroupedColumnLinear
+    p = GroupedColumnLinear(16, [[5, 3, 4], [8, 1], [2]], torch.float32)
+    assert [p.columns(i) for i in range(3)] == [(0, 12), (16, 25), (32, 34)] and p.weight.shape == (40, 16)
+    p.weight.data.fill_(float("nan"))
+    g = torch.Generator().manual_seed(1)
+    parts = {(i, j): torch.randn(n, 16, generator=g) for i, grp in enumerate([[5, 3, 4], [8, 1], [2]]) for j, n in enumerate(grp)}
+    for (i, j), w in parts.items():
+        p.weight_loader(p.weight, w, p.shard(i, j))
+    assert torch.isnan(p.weight).any()
+    p.finalize_weights()
+    x = torch.randn(3, 16, generator=g)
+    y = p(x)
+    for i in range(3):
+        lo, hi = p.columns(i)
+        want = torch.cat([x @ parts[(i, j)].T for j in range(len([k for k in parts if k[0] == i]))], 1)
+        assert torch.allclose(y[:, lo:hi], want, atol=1e-5)
+    assert y[:, 12:16].abs().max().item() == 0.0
+
+
+def test_config_errors():
+    from vllm_distributed_amd.models.bapovik import BapovikLayer
+    f32 = torch.float32
+    rank = {"l0.mix.right.a1": (4, 32), "l1.mix.right.a1": (4, 32)}
+    first = BapovikLayer(32, attention(4, 2, 8, 8, 9), 1e-5, 0, f32, rank, [])
+    par = BapovikLayer(32, parallel((4, 2, 8, 8, 9, 1.0, 2.0), (2, 8, 8, 4.0)), 1e-5, 0, f32, rank, [])
+    BapovikLayer(32, attention(4, 2, 8, 8, 90, kv_from=0), 1e-5, 1, f32, rank, [first])
+    assert first.mix.inner.attn.reach == 90
+    reader = BapovikLayer(32, attention(4, 2, 8, 8, 5, kv_from=0), 1e-5, 1, f32, rank, [first])
+    bad_mlp = attention(4, 2, 8, 8, 9, moe(4, 2, 8))
+    bad_mlp["mlp"]["kind"] = "other"
+    for bad, earlier in ((attention(4, 3, 8, 8, 9), [first]), (attention(4, 2, 8, 8, 9, kv_from=1), [first]),
+                         (attention(4, 2, 8, 8, 9, kv_from=-1), [first]), (attention(4, 2, 8, 12, 9, kv_from=0), [first]),
+                         (attention(4, 1, 8, 8, 9, kv_from=0), [first]), (attention(4, 2, 8, 8, 9, kv_from=0), [par]),
+                         (dict(attention(4, 2, 8, 8, 9), type="other"), [first]), (bad_mlp, [first]),
+                         (attention(4, 2, 8, 8, 9, moe(4, 5, 8)), [first])):
+        with pytest.raises(ValueError):
+            BapovikLayer(32, bad, 1e-5, 1, f32, rank, earlier)
+    with pytest.raises(ValueError):                            # a reader owns no keys another layer could read
+        BapovikLayer(32, attention(4, 2, 8, 8, 9, kv_from=1), 1e-5, 2, f32, rank, [first, reader])
+    with pytest.raises(ValueError):                            # the decay's narrow middle: stated nowhere
+        BapovikLayer(32, parallel((4, 2, 8, 8, 9, 1.0, 2.0), (2, 8, 8, 4.0)), 1e-5, 0, f32, {}, [])
+
+
+def test_a_missing_tensor_is_an_error(tmp_path_factory, tmp_path):
+    path, cfg, w = model_dir("degenerate", tmp_path_factory)
+    for name in ("l0.mix.right.a2.b", "l0.mix.left.out", "l1.mix.k.b", "l0.mlp.e0.up", "l4.mix.q.b", "l3.mix.left.g", "l2.norm1"):
+        assert name in w
+        d = tmp_path / name
+        d.mkdir()
+        save_model(d, cfg, {k: v for k, v in w.items() if k != name})
+        with pytest.raises(Exception):
+            run_schedule(str(d), [[("r", [1, 2], [1]), {"end": ["r"]}]], "float32", "cpu", max_tokens=64, tmp=tmp_path)
+
+
+def test_dummy_weights_and_config_keys():
+    """Random-weight loading (the benchmark's path): every parameter is filled, the derived keys are there."""
+    import tempfile
+    from vllm_distributed_amd import LLM, SamplingParams
+    from vllm_distributed_amd.config import normalize_hf_config
+    from vllm_distributed_amd.models.bapovik import weight_shapes
+    cfg = json.loads(json.dumps(CONFIGS["paged"]))
+    for spec in cfg["layers"]:
+        if spec["type"] == "parallel":
+            spec["mixer"]["right"]["decay_rank"] = 6
+    assert weight_shapes(cfg) == {k: tuple(v.shape) for k, v in random_weights(cfg, 1, 6).items()}
+    n = dict(cfg)
+    normalize_hf_config(n)
+    assert n["hidden_size"] == 64 and n["vocab_size"] == 97 and n["num_hidden_layers"] == 4 and n["num_attention_heads"] == 4
+    assert n["num_key_value_heads"] == 1 and n["head_dim"] == 16 and n["architectures"] == ["BapovikForCausalLM"]
+    with tempfile.TemporaryDirectory() as d:
+        with open(os.path.join(d, "config.json"), "w") as f:
+            json.dump(cfg, f)
+        llm = LLM(model=d, device="cpu", dtype="float32", max_model_len=64, max_num_seqs=2, block_size=16,
+                  load_format="dummy", enforce_eager=True)
+        try:
+            out = llm.generate([[1, 2, 3]], SamplingParams(temperature=0.0, max_tokens=4, ignore_eos=True))
+        finally:
+            llm.shutdown()
+        assert len(out[0].outputs[0].token_ids) == 4
+
+
+def test_the_bundled_configuration_runs():
+    from vllm_distributed_amd import LLM, SamplingParams
+    llm = LLM(model="bapovik-tiny", device="cpu", dtype="float32", max_model_len=128, max_num_seqs=2, block_size=16,
+              load_format="dummy", enforce_eager=True)
+    try:
+        out = llm.generate([list(range(70))], SamplingParams(temperature=0.0, max_tokens=4, ignore_eos=True))
+    finally:
+        llm.shutdown()
+    assert len(out[0].outputs[0].token_ids) == 4
+
+
+def test_the_trace_runner_as_a_program(tmp_path_factory, tmp_path):
+    import subprocess
+    import sys
+    path, cfg, w = model_dir("degenerate", tmp_path_factory)
+    a, b = tokens_for(cfg, 9, 50), tokens_for(cfg, 5, 51)
+    lines = [{"step": 0, "entries": [{"id": "a", "tokens": a[:6], "want": [0, 5]}, {"id": "b", "tokens": b[:2], "want": []}], "end": []},
+             {"step": 1, "entries": [{"id": "b", "tokens": b[2:], "want": []}], "end": ["b"]},
+             {"step": 2, "entries": [{"id": "a", "tokens": a[6:], "want": [2]}], "end": ["a"]}]
+    exe = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file__))), "bin", "trace_run")
+    r = subprocess.run([sys.executable, exe, "--model", path, "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "128",
+                        "--device", "cpu"], input="".join(json.dumps(x) + "\n" for x in lines), text=True,
+                       capture_output=True, timeout=300)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [l for l in r.stdout.splitlines() if l.startswith("done")] == ["done 0", "done 1", "done 2"]
+    want = oracle_logits(cfg, w, a)
+    got0 = np.fromfile(tmp_path / "0.f32", dtype="<f4").reshape(2, cfg["vocab"])
+    got2 = np.fromfile(tmp_path / "2.f32", dtype="<f4").reshape(1, cfg["vocab"])
+    assert np.abs(got0 - want[[0, 5]]).max() < 1e-4 and np.abs(got2 - want[[8]]).max() < 1e-4
+
+
+# ------------------------------------------------------------------------------------------- generation
+@pytest.mark.parametrize("device,dtype", OP_DEVICES)
+@pytest.mark.parametrize("name", ["varied", "windows"])
+def test_greedy_generation_through_the_scheduler(name, device, dtype, tmp_path_factory):
+    """``LLM.generate`` on five prompts with two sequence slots and small prefill chunks: the scheduler's own batching,
+    chunking and sampling.  Every generated token is the oracle's argmax given the tokens before it (in bfloat16: or
+    its logit is within rounding of the oracle's best)."""
+    from vllm_distributed_amd import LLM, SamplingParams
+    path, cfg, w = model_dir(name, tmp_path_factory, dtype)
+    prompts = [tokens_for(cfg, n, 40 + n) for n in (3, 30, 1, 17, 45)]
+    llm = LLM(model=path, device=device, dtype=dtype, max_model_len=128, max_num_seqs=2, max_num_batched_tokens=16,
+              block_size=16, load_format="safetensors", enforce_eager=False)
+    try:
+        outs = llm.generate(prompts, SamplingParams(temperature=0.0, max_tokens=24, ignore_eos=True))
+    finally:
+        llm.shutdown()
+    for prompt, o in zip(prompts, outs):
+        gen = list(o.outputs[0].token_ids)
+        assert len(gen) == 24
+        logits = oracle.forward(cfg, w, prompt + gen).numpy()
+        for i, tok in enumerate(gen):
+            row = logits[len(prompt) + i - 1]
+            if dtype == "float32":
+                assert tok == int(row.argmax()), (len(prompt), i)
+            else:
+                assert row.max() - row[tok] < 0.2, (len(prompt), i, float(row.max() - row[tok]))
