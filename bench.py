@@ -139,10 +139,11 @@ def _parse():
     ap.add_argument("--alt-parallelism", type=str, default="pp",
                     help="second layout measured in a child process after the headline when N > 1 ('none' = skip)")
     ap.add_argument("--alt-timeout", type=float, default=900.0)
-    ap.add_argument("--family-compare", type=str, default=None, choices=[None, "tavulix", "kabapel", "gosizen", "nalasun", "kefurax"],
+    ap.add_argument("--family-compare", type=str, default=None, choices=[None, "tavulix", "kabapel", "gosizen", "nalasun", "kefurax",
+                                                                              "bapovik"],
                     help="instead of the headline: prefill and decode throughput of this model family at a few layer "
                          "sizes beside the closest existing family at equal size (Tavulix: Gemma-2; Kabapel: "
-                         "DeepSeek-V2; Gosizen: Kabapel; Nalasun: Gosizen; Kefurax: Nalasun), random weights, one GPU")
+                         "DeepSeek-V2; Gosizen: Kabapel; Nalasun: Gosizen; Kefurax: Nalasun; Bapovik: Gosizen), random weights, one GPU")
     ap.add_argument("--compare-sizes", type=str, default="small,medium",
                     help="with --family-compare: which of small / medium / large to run")
     ap.add_argument("--compare-only", type=str, default=None,
@@ -347,6 +348,30 @@ def _kefurax_models(z: dict) -> dict:
     return {"kefurax": ("kefurax-tiny", kef), "nalasun": nal}
 
 
+def _bapovik_models(z: dict) -> dict:
+    """The same layer sizes as a Bapovik config (chunked attention beside gated linear attention, and windowed attention whose
+    second layer reads the first one's keys, in turn; an expert block in every layer) and as a Gosizen config (chunked attention
+    beside the gated delta rule, windowed latent attention, expert blocks, mixer and feed-forward side by side on one
+    normed input around an fp32 residual stream: the closest family the framework has)."""
+    vocab = 32000
+    moe = {"kind": "moe", "expert": {"ff": z["ff"]}, "router": {"experts": z["experts"] + z["identity"], "top": z["top"]}}
+    window, kv = min(z["prompt"], 1024), max(z["heads"] // 4, 1)
+    att = {"heads": z["heads"], "kv_heads": kv, "dim": z["nope"], "vdim": z["vdim"], "scale": z["nope"] ** -0.5,
+           "mask": {"size": window}}
+    par = {"left": dict(att, softcap=50.0),
+           "right": {"heads": z["heads"], "dim": z["nope"], "vdim": z["vdim"], "tau": 16.0, "decay_rank": 16}}
+    layers, first = [], None
+    for i in range(z["layers"]):
+        if i % 2 == 0:
+            layers.append({"type": "parallel", "mixer": par, "mlp": moe})
+        else:
+            m = dict(att) if first is None else dict(att, kv_from=first)
+            first = i if first is None else first
+            layers.append({"type": "attention", "mixer": m, "mlp": moe})
+    bap = {"architecture": "Bapovik", "vocab": vocab, "width": z["width"], "norm": {"eps": 1e-6}, "layers": layers}
+    return {"bapovik": ("bapovik-tiny", bap), "gosizen": _gosizen_models(z)["gosizen"]}
+
+
 def run_family_compare(args) -> None:
     """Prefill throughput (``prompts`` prompts of ``prompt`` tokens, one generated token each) and decode
     throughput (``batch`` sequences, 64 further tokens each; the prefill time measured the same way is taken off)
@@ -356,11 +381,11 @@ def run_family_compare(args) -> None:
     from vllm_distributed_amd import LLM, SamplingParams
     os.environ.setdefault("VLLM_LOGGING_LEVEL", "WARNING")
     rows = []
-    kabapel = args.family_compare in ("kabapel", "gosizen", "nalasun", "kefurax")
+    kabapel = args.family_compare in ("kabapel", "gosizen", "nalasun", "kefurax", "bapovik")
     for size in [s for s in args.compare_sizes.split(",") if s]:
         z = (KABAPEL_SIZES if kabapel else COMPARE_SIZES)[size]
         by_family = {"gosizen": _gosizen_models, "nalasun": _nalasun_models, "kabapel": _kabapel_models,
-                     "kefurax": _kefurax_models}
+                     "kefurax": _kefurax_models, "bapovik": _bapovik_models}
         models = by_family[args.family_compare](z) if kabapel else _compare_models(z)
         for family, (base, over) in models.items():
             if args.compare_only and family != args.compare_only:

@@ -433,16 +433,26 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(NW >= 1
   if (e <= s) return;                                            // (uniform over the workgroup)
   const bool fresh = seq_lens[b] - (e - s) <= 0;                 // whatever the slot holds is not ours
   float* st = state + ((long)slots[b] * H + h) * (long)dim * vdim;
-  const bool pair = (vdim & 1) == 0;                             // (both columns of a lane exist or none, 8-byte aligned)
+  // the lane's part of the state is there whole (both columns, every row; 8-byte aligned): its accesses carry no conditions
+  // and are all in flight together
+  const bool whole = (vdim & 1) == 0 && row0 + R <= dim && c0 < vdim;
   float S0[R], S1[R];
 #pragma unroll
-  for (int i = 0; i < R; ++i) {
-    const int r = row0 + i;
-    S0[i] = S1[i] = 0.f;
-    if (!fresh && r < dim && c0 < vdim) {
-      const float* p = st + (long)r * vdim + c0;
-      if (pair) { const float2 f = *reinterpret_cast<const float2*>(p); S0[i] = f.x; S1[i] = f.y; }
-      else { S0[i] = p[0]; if (c0 + 1 < vdim) S1[i] = p[1]; }
+  for (int i = 0; i < R; ++i) S0[i] = S1[i] = 0.f;
+  if (!fresh) {
+    if (whole) {
+#pragma unroll
+      for (int i = 0; i < R; ++i) {
+        const float2 f = *reinterpret_cast<const float2*>(st + (long)(row0 + i) * vdim + c0);
+        S0[i] = f.x;
+        S1[i] = f.y;
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < R; ++i) {
+        const float* p = st + (long)(row0 + i) * vdim + c0;
+        if (row0 + i < dim && c0 < vdim) { S0[i] = p[0]; if (c0 + 1 < vdim) S1[i] = p[1]; }
+      }
     }
   }
   const long qoff = (long)h * dim, koff = (long)(H + h) * dim, voff = 2L * H * dim + (long)h * vdim;
@@ -517,13 +527,15 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(NW >= 1
       }
     }
   }
+  if (whole) {
 #pragma unroll
-  for (int i = 0; i < R; ++i) {
-    const int r = row0 + i;
-    if (r < dim && c0 < vdim) {
-      float* p = st + (long)r * vdim + c0;
-      if (pair) *reinterpret_cast<float2*>(p) = make_float2(S0[i], S1[i]);
-      else { p[0] = S0[i]; if (c0 + 1 < vdim) p[1] = S1[i]; }
+    for (int i = 0; i < R; ++i)
+      *reinterpret_cast<float2*>(st + (long)(row0 + i) * vdim + c0) = make_float2(S0[i], S1[i]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+      float* p = st + (long)(row0 + i) * vdim + c0;
+      if (row0 + i < dim && c0 < vdim) { p[0] = S0[i]; if (c0 + 1 < vdim) p[1] = S1[i]; }
     }
   }
 }
@@ -948,12 +960,14 @@ VDAMD_API int vdamd_channel_decay_attention(float* out, const void* x, long x_st
 #define CDA(R_, NW_, C_)                                                                                              \
   hipLaunchKernelGGL((channel_decay_attention_kernel<TT, R_, NW_, C_>), grid, dim3(64 * NW_), 0, stream, out,          \
                      (const TT*)x, x_stride, alpha, state, slots, qsl, seq_lens, H, dim, vdim, scale, silu)
-    if (max_rows > 0 && max_rows <= 2) {                         // decoded rows: bound by the states, small workgroups
+    // Decoded rows are bound by reading and writing the states, many sequences by issue: small workgroups, several of
+    // which fit a CU and fill each other's waits.  Few sequences are bound by the walk over the rows: large workgroups.
+    if ((max_rows > 0 && max_rows <= 2) || (long)grid.x * grid.y * grid.z >= 512) {
       if (dim <= 32) CDA(4, 4, 8);
       else if (dim <= 64) CDA(8, 4, 4);
       else if (dim <= 128) CDA(16, 4, 4);
       else CDA(32, 4, 4);
-    } else {                                                     // prompt portions: bound by the walk over the rows
+    } else {
       if (dim <= 32) CDA(4, 4, 8);
       else if (dim <= 64) CDA(4, 8, 8);
       else if (dim <= 128) CDA(4, 16, 8);

@@ -88,15 +88,20 @@ __global__ void residual_rms_kernel(ResidualArgs p) {
   const TA* yr = p.y ? (const TA*)p.y + row * p.y_stride : nullptr;
   const TA* zr = p.z ? (const TA*)p.z + row * p.z_stride : nullptr;
   const int n = p.H / W;
-  auto inv_rms = [&](const TA* r) {                 // post_scale / rms of a row
-    float ss = 0.f;
+  float inv_y = 0.f, inv_z = 0.f;
+  if (yr != nullptr) {
+    auto square = [&](const TA* r, int i) {
+      if constexpr (W == 4) { const f32x4 v = ld4<TA>(r + 4 * i); return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
+      else { const float v = ldf(r + i); return v * v; }
+    };
+    float sy = 0.f, sz = 0.f;
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
-      if constexpr (W == 4) { const f32x4 v = ld4<TA>(r + 4 * i); ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
-      else { const float v = ldf(r + i); ss += v * v; }
+      sy += square(yr, i);
+      if (zr != nullptr) sz += square(zr, i);
     }
-    return p.post_scale / sqrtf(block_sum(ss, red) / (float)p.H + p.eps);
-  };
-  const float inv_y = yr != nullptr ? inv_rms(yr) : 0.f, inv_z = zr != nullptr ? inv_rms(zr) : 0.f;
+    inv_y = p.post_scale / sqrtf(block_sum(sy, red) / (float)p.H + p.eps);
+    if (zr != nullptr) inv_z = p.post_scale / sqrtf(block_sum(sz, red) / (float)p.H + p.eps);
+  }
   const bool adds = ar != nullptr || yr != nullptr;
   float ss = 0.f;
   for (int i = threadIdx.x; i < n; i += blockDim.x) {

@@ -723,6 +723,18 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_kernel(RotArgs a) {
   }
 }
 
+// eight fp32 values at p + off (16-byte aligned), or `otherwise` without p: one branch and two loads, not eight of each
+__device__ __forceinline__ void rot_eight(const float* p, long off, float otherwise, float (&o)[8]) {
+  if (p != nullptr) {
+    const f32x4 lo = *reinterpret_cast<const f32x4*>(p + off), hi = *reinterpret_cast<const f32x4*>(p + off + 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { o[e] = lo[e]; o[e + 4] = hi[e]; }
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) o[e] = otherwise;
+  }
+}
+
 // 16-bit types, neighbouring pairs, head sizes of 8 L with L a power of two: a lane owns 8 channels (4 pairs) of a head,
 // the sum of squares over the head's L neighbouring lanes by xor-shuffles
 template <typename T>
@@ -740,13 +752,16 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_vec_kernel(RotArgs a, i
   for (int idx = threadIdx.x; idx < (a.H + a.G) * L; idx += blockDim.x) {
     const int u = idx >> sh, d = (idx & (L - 1)) * 8;
     const V8 xv = ld8<T>(xr + (long)u * a.D + d);
-    const float* b = a.bias ? a.bias + (long)u * a.D + d : nullptr;
-    float v[8];
+    const bool is_q = u < a.H;
+    const float* w = is_q ? a.q_norm : a.k_norm;
+    float v[8], bf[8], wf[8];
+    rot_eight(a.bias, (long)u * a.D + d, 0.f, bf);
+    rot_eight(w, d, 1.f, wf);
     float ss = 0.f;
 #pragma unroll
     for (int e = 0; e < 8; e += 2) {
       const int i = (d + e) >> 1;
-      const float p = (float)xv[e] + (b ? b[e] : 0.f), q = (float)xv[e + 1] + (b ? b[e + 1] : 0.f);
+      const float p = (float)xv[e] + bf[e], q = (float)xv[e + 1] + bf[e + 1];
       const bool rot = i < a.half;
       const float c = rot ? cs[i] : 1.f, s = rot ? sn[i] : 0.f;
       v[e] = p * c - q * s;
@@ -758,11 +773,9 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_vec_kernel(RotArgs a, i
       for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
       inv = 1.0f / sqrtf(ss / (float)a.D + a.eps);
     }
-    const bool is_q = u < a.H;
-    const float* w = is_q ? a.q_norm : a.k_norm;
     V8 r;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) r[e] = (T)(v[e] * inv * (w ? w[d + e] : 1.f));
+    for (int e = 0; e < 8; ++e) r[e] = (T)(v[e] * inv * wf[e]);
     if (is_q) st8<T>((T*)a.q_out + (t * a.H + u) * (long)a.D + d, r);
     else if (slot >= 0) st8<T>((T*)a.k_cache + ((blk * a.G + (u - a.H)) * a.bs + off) * (long)a.D + d, r);
   }
@@ -772,7 +785,8 @@ __global__ __launch_bounds__(256) void rotate_norm_cache_vec_kernel(RotArgs a, i
     const int g = i / a.Dv, d = i - g * a.Dv;                     // (Dv % 8 == 0: the 8 channels share a head)
     V8 vv = ld8<T>(vr + i);
     if (a.bias) {
-      const float* vb = a.bias + (long)(a.H + a.G) * a.D + i;
+      float vb[8];
+      rot_eight(a.bias, (long)(a.H + a.G) * a.D + i, 0.f, vb);
 #pragma unroll
       for (int e = 0; e < 8; ++e) vv[e] = (T)((float)vv[e] + vb[e]);
     }
@@ -1379,7 +1393,8 @@ VDAMD_API int vdamd_rotate_norm_cache(void* q_out, const void* x, long x_stride,
   const int L = D / 8;
   auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
   const bool vec = dt != DT_F32 && (interleaved || half == 0) && D % 8 == 0 && (L & (L - 1)) == 0 && L <= 64 &&
-                   Dv % 8 == 0 && x_stride % 8 == 0 && al16(x) && al16(q_out) && al16(k_cache);
+                   Dv % 8 == 0 && x_stride % 8 == 0 && al16(x) && al16(q_out) && al16(k_cache) && al16(bias) && al16(q_norm) &&
+                   al16(k_norm);
   return by_dtype(dt, [&](auto* tp) {
     using TT = std::remove_pointer_t<decltype(tp)>;
     if constexpr (!std::is_same_v<TT, float>) {

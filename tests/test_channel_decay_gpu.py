@@ -77,6 +77,20 @@ def test_channel_decay_attention(dtype, heads, dim, vdim):
             _close(hip.decay_linear_attention(x, heads, dim, vdim, alpha, s1, slots, qsl, lens, silu, 0, 0.3), want, 1e-5)
 
 
+@pytest.mark.parametrize("heads,dim,vdim", [(8, 20, 70), (8, 64, 64), (4, 128, 128), (8, 130, 32)])
+def test_many_sequences_in_one_launch(heads, dim, vdim):
+    """Enough workgroups for the launch shape of crowded prompt steps: portions of one to nine rows."""
+    hip = _hip()
+    sizes = [1 + (7 * i) % 9 for i in range(66)]
+    starts = [(5 * i) % 4 for i in range(66)]
+    x, alpha, state, slots, qsl, lens = _recurrence(heads, dim, vdim, sizes, starts, torch.bfloat16, dim)
+    s1, s2 = state.clone(), state.clone()
+    got = hip.decay_linear_attention(x, heads, dim, vdim, alpha, s1, slots, qsl, lens, False, 9, 0.5)
+    want = torch_ref.decay_linear_attention(x, heads, dim, vdim, alpha, s2, slots, qsl, lens, False, 0.5)
+    _close(got, want, 1e-5)
+    _close(s1, s2, 1e-5)
+
+
 @pytest.mark.parametrize("heads,dim,vdim", [(2, 64, 64), (1, 128, 128), (3, 24, 40)])
 def test_portions_leave_the_state_a_whole_pass_leaves(heads, dim, vdim):
     hip = _hip()

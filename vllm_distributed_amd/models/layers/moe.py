@@ -576,7 +576,10 @@ class PlainTopKMoE(FusedMoE):
         if self.num_experts > 512 or self.top_k > 16 or self.hidden % 16:
             return 0
         avg = x.shape[0] * self.top_k / max(1, self.num_experts)
-        if avg > envs.VDAMD_MOE_GROUPED_MAX_ROWS * 2 and not torch.cuda.is_current_stream_capturing():
+        # one library GEMM per expert pays for its host synchronisation and scattered sums only where the experts are large
+        # (2048 rows each: 4096 x 1408 experts take 0.89 ms grouped and 1.38 ms one by one, 4096 x 8192 ones 3.8 and 3.0)
+        if (avg > envs.VDAMD_MOE_GROUPED_MAX_ROWS * 2 and self.hidden * self.inter >= 12 << 20
+                and not torch.cuda.is_current_stream_capturing()):
             return 0
         for rows in (16, 32, 64, 128):
             if avg <= rows:
