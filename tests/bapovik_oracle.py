@@ -88,11 +88,13 @@ def window_mixer(h, w, p, m, eps, kept):
     return attend(h, q, k, v, w, p, m, window_mask(t, int(m["mask"]["size"])))
 
 
-def chunked_half(h, w, p, m, eps):
+def chunked_half(h, w, p, m, eps, kept=None):
     t = h.shape[0]
     q = project(h, w, p + "q").view(t, int(m["heads"]), int(m["dim"]))
     k, v = keys_values(h, w, p, m)
     q, k = unit_rms(q, eps) * f64(w[p + "q.norm"]), unit_rms(k, eps) * f64(w[p + "k.norm"])
+    if kept is not None:
+        kept[int(p[1:].split(".")[0])] = (k, v)
     return attend(h, q, k, v, w, p, m, chunk_mask(t, int(m["mask"]["size"])), float(m["softcap"]), True)
 
 
@@ -124,8 +126,8 @@ def recurrent_half(h, w, p, m, eps):
     return (o * silu(h @ f64(w[p + "g"]).T)) @ f64(w[p + "o"]).T
 
 
-def parallel_mixer(h, w, p, m, eps):
-    left = chunked_half(h, w, p + "left.", m["left"], eps)
+def parallel_mixer(h, w, p, m, eps, kept=None):
+    left = chunked_half(h, w, p + "left.", m["left"], eps, kept)
     right = recurrent_half(h, w, p + "right.", m["right"], eps)
     return 0.5 * (unit_rms(left, eps) * f64(w[p + "left.out"]) + unit_rms(right, eps) * f64(w[p + "right.out"]))
 
@@ -157,7 +159,7 @@ def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens: List[int], residuals:
         p, m = f"l{i}.", spec["mixer"]
         h = unit_rms(x, eps) * f64(w[p + "norm1"])
         if spec["type"] == "parallel":
-            y = parallel_mixer(h, w, p + "mix.", m, eps)
+            y = parallel_mixer(h, w, p + "mix.", m, eps, kept)
         else:
             y = window_mixer(h, w, p + "mix.", m, eps, kept)
         if spec.get("mlp"):

@@ -68,12 +68,13 @@ CONFIGS = {
         attention(2, 2, 8, 8, 500),
         parallel((2, 2, 8, 8, 400, 1.0, 30.0), (1, 8, 8, 1.0), moe(2, 1, 16)),
         attention(2, 2, 8, 8, 1, None, kv_from=2)], width=32, vocab=50),
-    # masks and sequences over several pages of 16 tokens
+    # masks and sequences over several pages of 16 tokens; a window over the keys of a parallel layer's left half
     "paged": config([
         parallel((4, 1, 16, 16, 40, 1.1, 6.0), (4, 16, 16, 8.0), moe(8, 2, 32)),
         attention(4, 4, 16, 24, 33, moe(4, 1, 32)),
         attention(4, 4, 16, 24, 49, moe(4, 2, 16), kv_from=1),
-        parallel((2, 2, 32, 24, 48, 0.8, 20.0), (2, 20, 32, 16.0))], width=64),
+        parallel((2, 2, 32, 24, 48, 0.8, 20.0), (2, 20, 32, 16.0)),
+        attention(4, 1, 16, 16, 60, None, kv_from=0)], width=64),
     # sizes the 16-bit kernels' 16-byte and matrix-core paths take
     "wide": config([
         attention(8, 2, 32, 64, 40, moe(6, 2, 128)),
@@ -727,12 +728,14 @@ def test_config_errors():
     par = BapovikLayer(32, parallel((4, 2, 8, 8, 9, 1.0, 2.0), (2, 8, 8, 4.0)), 1e-5, 0, f32, rank, [])
     BapovikLayer(32, attention(4, 2, 8, 8, 90, kv_from=0), 1e-5, 1, f32, rank, [first])
     assert first.mix.inner.attn.reach == 90
+    BapovikLayer(32, attention(4, 2, 8, 8, 50, kv_from=0), 1e-5, 1, f32, rank, [par])
+    assert par.heads.attn.reach == 50 and par.heads.attn.chunk == 9
     reader = BapovikLayer(32, attention(4, 2, 8, 8, 5, kv_from=0), 1e-5, 1, f32, rank, [first])
     bad_mlp = attention(4, 2, 8, 8, 9, moe(4, 2, 8))
     bad_mlp["mlp"]["kind"] = "other"
     for bad, earlier in ((attention(4, 3, 8, 8, 9), [first]), (attention(4, 2, 8, 8, 9, kv_from=1), [first]),
                          (attention(4, 2, 8, 8, 9, kv_from=-1), [first]), (attention(4, 2, 8, 12, 9, kv_from=0), [first]),
-                         (attention(4, 1, 8, 8, 9, kv_from=0), [first]), (attention(4, 2, 8, 8, 9, kv_from=0), [par]),
+                         (attention(4, 1, 8, 8, 9, kv_from=0), [first]), (attention(4, 4, 8, 8, 9, kv_from=0), [par]),
                          (dict(attention(4, 2, 8, 8, 9), type="other"), [first]), (bad_mlp, [first]),
                          (attention(4, 2, 8, 8, 9, moe(4, 5, 8)), [first])):
         with pytest.raises(ValueError):
@@ -767,7 +770,7 @@ def test_dummy_weights_and_config_keys():
     assert weight_shapes(cfg) == {k: tuple(v.shape) for k, v in random_weights(cfg, 1, 6).items()}
     n = dict(cfg)
     normalize_hf_config(n)
-    assert n["hidden_size"] == 64 and n["vocab_size"] == 97 and n["num_hidden_layers"] == 4 and n["num_attention_heads"] == 4
+    assert n["hidden_size"] == 64 and n["vocab_size"] == 97 and n["num_hidden_layers"] == 5 and n["num_attention_heads"] == 4
     assert n["num_key_value_heads"] == 1 and n["head_dim"] == 16 and n["architectures"] == ["BapovikForCausalLM"]
     with tempfile.TemporaryDirectory() as d:
         with open(os.path.join(d, "config.json"), "w") as f:

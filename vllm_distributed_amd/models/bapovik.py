@@ -8,7 +8,8 @@ give fp32 logits.  Positions enter nowhere but through the masks and the recurre
 
 Mixers
   * ``attention`` - ``GatedHeads``: q, k and v with biases, a sliding window, an ordinary softmax, a sigmoid gate per head.  A
-    layer with ``kv_from: j`` has no keys and values: it reads what layer ``j`` cached, with its own queries and mask.
+    layer with ``kv_from: j`` has no keys and values: it reads what layer ``j`` cached (a parallel layer: its left half),
+    with its own queries and mask.
   * ``parallel`` - ``layers.parallel_heads.ParallelNormed``: two mixers side by side on the same input, each one's output
     RMS-normed, half their sum.  left = ``GatedHeads`` with a head norm on q and k, scores squashed to
     ``cap tanh(s / cap)``, a mask of blocks of positions counted from the sequence's start, one added to the softmax
@@ -100,9 +101,9 @@ class GatedHeads(nn.Module):
 
 class AttentionMixer(nn.Module):
     def __init__(self, width: int, m: dict, eps: float, layer_idx: int, dtype: torch.dtype,
-                 source: Optional["AttentionMixer"]):
+                 source: Optional[GatedHeads]):
         super().__init__()
-        self.inner = GatedHeads(m, eps, layer_idx, source=None if source is None else source.inner)
+        self.inner = GatedHeads(m, eps, layer_idx, source=source)
         self.proj = GroupedColumnLinear(width, [self.inner.sizes], dtype)
         self.o = RowParallelLinear(self.inner.out_cols, width, False, dtype)
 
@@ -135,9 +136,9 @@ class BapovikLayer(nn.Module):
             source = None
             if m.get("kv_from") is not None:
                 j = int(m["kv_from"])
-                if not 0 <= j < layer_idx or not isinstance(earlier[j].mix, AttentionMixer):
-                    raise ValueError(f"layer {layer_idx}: kv_from {j} names no earlier attention layer")
-                source = earlier[j].mix
+                if not 0 <= j < layer_idx:
+                    raise ValueError(f"layer {layer_idx}: kv_from {j} names no earlier layer")
+                source = earlier[j].heads
             self.mix = AttentionMixer(width, m, eps, layer_idx, dtype, source)
         elif kind == "parallel":
             self.mix = _parallel(width, m, eps, layer_idx, dtype, shapes)
@@ -151,6 +152,11 @@ class BapovikLayer(nn.Module):
             self.mlp = PlainTopKMoE(width, int(mlp["expert"]["ff"]), int(mlp["router"]["experts"]),
                                     int(mlp["router"]["top"]), dtype, activation="relu2", scores="sigmoid",
                                     weigh_input=True)
+
+    @property
+    def heads(self) -> GatedHeads:
+        """The layer's softmax attention (of a parallel mixer: its left half)."""
+        return self.mix.left if isinstance(self.mix, ParallelNormed) else self.mix.inner
 
     def forward(self, x: torch.Tensor, h: torch.Tensor, then: ResidualRMSNorm) -> torch.Tensor:
         """``x``: fp32 residual stream (updated in place), ``h = norm1(x)``; returns ``then(x)`` after this layer.  The
@@ -198,8 +204,7 @@ class BapovikForCausalLM(nn.Module):
 
     def attention_layers(self) -> List[Attention]:
         """The layers that own keys and values (a layer that reads another's owns none)."""
-        attns = [l.mix.left.attn if isinstance(l.mix, ParallelNormed) else l.mix.inner.attn for l in self.layers]
-        return [a for a in attns if a.source is None]
+        return [l.heads.attn for l in self.layers if l.heads.attn.source is None]
 
     def state_layers(self) -> List[SlotState]:
         return [l.mix.right.slot_state for l in self.layers if isinstance(l.mix, ParallelNormed)]
